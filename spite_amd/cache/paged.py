@@ -33,7 +33,7 @@ class OutOfPages(CacheError):
 
 @dataclass
 class Group:
-    key: tuple                   # (kv heads, key width, visibility, span, value width, value heads)
+    key: tuple                   # (kv heads, key width, visibility, span, value width, value heads, first positions kept)
     cache_ids: List[int]
     n_pages: int
     k: Optional[torch.Tensor] = None     # [layers, pages, G, page_size, key width]
@@ -61,8 +61,9 @@ class PagedCache:
             if need is None or need.kv is None:
                 continue
             kv = need.kv
-            key = (kv.n_kv_heads, kv.head_dim, kv.visibility, kv.span if kv.visibility != "full" else 0, kv.value_dim,
-                   kv.value_heads)
+            local = kv.visibility != "full"
+            key = (kv.n_kv_heads, kv.head_dim, kv.visibility, kv.span if local else 0, kv.value_dim, kv.value_heads,
+                   kv.keep if local else 0)
             if key not in by_key:
                 by_key[key] = len(self.groups)
                 self.groups.append(Group(key, [], 0, None))
@@ -80,9 +81,10 @@ class PagedCache:
         self._lib = lib
         kinds = hostlib.int_array(_KINDS[g.key[2]] for g in self.groups)
         spans = hostlib.int_array(g.key[3] for g in self.groups)
+        keeps = hostlib.int_array(g.key[6] for g in self.groups)
 
         def create():
-            h = lib.spc_create(self.page_size, self.max_requests, n_groups, kinds, spans, hostlib.int_array(pages))
+            h = lib.spc_create(self.page_size, self.max_requests, n_groups, kinds, spans, hostlib.int_array(pages), keeps)
             if not h:
                 raise CacheError(hostlib.last_error())
             return h
@@ -228,9 +230,9 @@ class PagedCache:
 
     def kv_tiled(self, cache_id: int) -> bool:
         """Whether this cache's pages are kept in the MFMA attention kernels' operand order
-        (bfloat16, head size and page size multiples of 32) rather than row-major."""
+        (bfloat16, key width, value width and page size multiples of 32) rather than row-major."""
         g = self.groups[self._group_of[cache_id]]
-        return g.key[1] == g.key[4] and hipops.kv_tiled_ok(self.dtype, g.key[1], self.page_size)
+        return g.key[4] > 0 and all(hipops.kv_tiled_ok(self.dtype, w, self.page_size) for w in (g.key[1], g.key[4]))
 
     def layer_pages(self, cache_id: int):
         g = self.groups[self._group_of[cache_id]]

@@ -24,17 +24,19 @@
 #include "common.h"
 #include "no_alloc.h"
 
-template <int HD>
+// HD: width of queries and keys, VD: of values.  DIST: the scores take a bias by distance from a table.
+template <int HD, int VD, bool DIST>
 __global__ __launch_bounds__(256)
 void attn_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_pages,
                         const bf16* __restrict__ v_pages, float* __restrict__ part, bf16* __restrict__ out,
                         const int* __restrict__ positions, const int* __restrict__ seq_of_token,
                         const int* __restrict__ block_table, int max_blocks, int H, int G, int ps, int vis,
                         int span, float scale_log2e, float cap_ratio, int n_splits,
-                        const float* __restrict__ slopes, float inv_scale, int Gv, const float* __restrict__ sinks) {
+                        const float* __restrict__ slopes, float inv_scale, int Gv, const float* __restrict__ sinks,
+                        int keep, const float* __restrict__ dist_bias, int n_dist) {
     constexpr int NC = HD / 32;      // 32-wide chunks of the head for the score product
-    constexpr int ND = HD / 16;      // 16-row tiles of the output
-    constexpr int ROW = HD + 2;      // partial record: output, max, sum
+    constexpr int ND = VD / 16;      // 16-row tiles of the output
+    constexpr int ROW = VD + 2;      // partial record: output, max, sum
     extern __shared__ float sm[];    // [4 waves][16 heads][ROW]
     const int split = blockIdx.x, g = blockIdx.y, t = blockIdx.z;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -46,11 +48,18 @@ void attn_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_p
     // a bias slope * (key - query position) on the scaled score of head n, as an addend of the raw score
     const float slope = (slopes && n < QH) ? slopes[g * QH + n] * inv_scale : 0.f;
 
+    // with a bias by distance: the table row of head n (added to the raw score, so divided by the scale), the same
+    // number for every distance from n_dist - 1 on
+    const float* tab = DIST ? dist_bias + (size_t)(g * QH + (n < QH ? n : 0)) * n_dist : nullptr;
+    const float far_bias = DIST ? tab[n_dist - 1] * inv_scale : 0.f;
+
+    // the blocks of the kept first keys (they stay in sight below the rule's first key), then the rule's own
     const int b_first = lo / 32, b_last = p / 32;
-    const int nblk = b_last - b_first + 1;
+    const int b_kept = min((keep + 31) / 32, b_first);
+    const int nblk = b_kept + b_last - b_first + 1;
     const int per = (nblk + n_splits - 1) / n_splits;
-    const int rb = b_first + split * per;
-    const int re = (rb + per < b_last + 1) ? rb + per : b_last + 1;
+    const int rb = split * per;
+    const int re = (rb + per < nblk) ? rb + per : nblk;
 
     const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
     bf16x8 qf[NC];
@@ -66,15 +75,15 @@ void attn_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_p
 #pragma unroll
     for (int d = 0; d < ND; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-    for (int kb = rb + wave; kb < re; kb += 4) {
-        const int key0 = kb * 32;
+    for (int i = rb + wave; i < re; i += 4) {
+        const int key0 = (i < b_kept ? i : b_first + (i - b_kept)) * 32;
         const int page = bt[key0 / ps];
         const int off0 = key0 % ps;
         const size_t pg = (size_t)(page < 0 ? 0 : page) * G + g;
         const int blk = off0 >> 5;                                   // the block of 32 keys inside the page
         const bf16* kbase = k_pages + pg * ps * HD + (size_t)blk * 2 * NC * 512 + lane * 8;
         // (value heads may be fewer than key heads: key head g reads value head g % Gv)
-        const bf16* vbase = v_pages + ((size_t)(page < 0 ? 0 : page) * Gv + g % Gv) * HD * ps + (size_t)blk * ND * 512 + lane * 8;
+        const bf16* vbase = v_pages + ((size_t)(page < 0 ? 0 : page) * Gv + g % Gv) * VD * ps + (size_t)blk * ND * 512 + lane * 8;
         bf16x8 kf[2][NC];
 #pragma unroll
         for (int tt = 0; tt < 2; ++tt)
@@ -106,13 +115,15 @@ void attn_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_p
         }
         float mx = -INFINITY;
         bool ok[2][4];
+        const bool near = DIST && key0 + 31 > p - (n_dist - 1);      // some key of the block is nearer than the table's end
 #pragma unroll
         for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int j = key0 + qd * 8 + tt * 4 + i;
-                ok[tt][i] = j >= lo && j <= p;
+                ok[tt][i] = sp_visible(j, p, lo, keep);
                 float raw = s[tt][i] + slope * (float)(j - p);
+                if (DIST) raw += near ? tab[min(max(p - j, 0), n_dist - 1)] * inv_scale : far_bias;
                 // a cap on the scores: cap * tanh(score * scale / cap), with cap_ratio = scale / cap
                 if (cap_ratio > 0.f) raw = tanhf(raw * cap_ratio) / cap_ratio;
                 const float v = ok[tt][i] ? (page < 0 ? NAN : raw * scale_log2e) : -INFINITY;
@@ -148,23 +159,23 @@ void attn_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_p
     for (int d = 0; d < ND; ++d)
 #pragma unroll
         for (int i = 0; i < 4; ++i) mine[d * 16 + qd * 4 + i] = o[d][i];
-    if (qd == 0) { mine[HD] = m_run; mine[HD + 1] = l_run; }
+    if (qd == 0) { mine[VD] = m_run; mine[VD + 1] = l_run; }
     __syncthreads();
     if (n_splits == 1) {                 // nothing to combine: the four waves' sums are the result
-        for (int idx = threadIdx.x; idx < QH * HD; idx += 256) {
-            const int hn = idx / HD, c = idx % HD;
+        for (int idx = threadIdx.x; idx < QH * VD; idx += 256) {
+            const int hn = idx / VD, c = idx % VD;
             float M = -INFINITY;
 #pragma unroll
-            for (int w = 0; w < 4; ++w) M = fmaxf(M, sm[((size_t)w * 16 + hn) * ROW + HD]);
+            for (int w = 0; w < 4; ++w) M = fmaxf(M, sm[((size_t)w * 16 + hn) * ROW + VD]);
             float acc = 0.f, L = 0.f;
 #pragma unroll
             for (int w = 0; w < 4; ++w) {
-                const float mw = sm[((size_t)w * 16 + hn) * ROW + HD];
+                const float mw = sm[((size_t)w * 16 + hn) * ROW + VD];
                 const float f = (mw == -INFINITY) ? 0.f : exp2f(mw - M);
                 acc += f * sm[((size_t)w * 16 + hn) * ROW + c];
-                L += f * sm[((size_t)w * 16 + hn) * ROW + HD + 1];
+                L += f * sm[((size_t)w * 16 + hn) * ROW + VD + 1];
             }
-            out[((size_t)t * H + g * QH + hn) * HD + c] = (bf16)(acc * (1.0f / fmaxf(L, 1e-30f)));
+            out[((size_t)t * H + g * QH + hn) * VD + c] = (bf16)(acc * (1.0f / fmaxf(L, 1e-30f)));
         }
         return;
     }
@@ -172,23 +183,23 @@ void attn_decode_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_p
         const int hn = idx / ROW, c = idx % ROW;
         float M = -INFINITY;
 #pragma unroll
-        for (int w = 0; w < 4; ++w) M = fmaxf(M, sm[((size_t)w * 16 + hn) * ROW + HD]);
+        for (int w = 0; w < 4; ++w) M = fmaxf(M, sm[((size_t)w * 16 + hn) * ROW + VD]);
         float acc = 0.f;
-        if (c == HD) acc = M;
+        if (c == VD) acc = M;
         else {
 #pragma unroll
             for (int w = 0; w < 4; ++w) {
-                const float mw = sm[((size_t)w * 16 + hn) * ROW + HD];
+                const float mw = sm[((size_t)w * 16 + hn) * ROW + VD];
                 const float f = (mw == -INFINITY) ? 0.f : exp2f(mw - M);
-                acc += f * sm[((size_t)w * 16 + hn) * ROW + c];   // c == HD+1 sums the l's
+                acc += f * sm[((size_t)w * 16 + hn) * ROW + c];   // c == VD+1 sums the l's
             }
         }
         part[(((size_t)t * H + g * QH + hn) * n_splits + split) * ROW + c] = acc;
     }
 }
 
-template <int HD>
-__global__ __launch_bounds__(HD)
+template <int HD>              // HD: the values' width
+__global__ __launch_bounds__(HD < 64 ? 64 : HD)
 void attn_decode_combine_kernel(const float* __restrict__ part, bf16* __restrict__ out, int H, int n_splits) {
     constexpr int ROW = HD + 2;
     __shared__ float wsh[256];          // weight of every split: exp2(m_s - M)
@@ -219,6 +230,7 @@ void attn_decode_combine_kernel(const float* __restrict__ part, bf16* __restrict
         if (c == 0) linv = 1.0f / fmaxf(L, 1e-30f);
     }
     __syncthreads();
+    if (c >= HD) return;                // (narrow values: one wave, not all of its lanes hold an element)
     float acc = 0.f;
 #pragma unroll 8
     for (int s = 0; s < n_splits; ++s) acc += wsh[s] * rec[(size_t)s * ROW + c];
@@ -226,57 +238,60 @@ void attn_decode_combine_kernel(const float* __restrict__ part, bf16* __restrict
 }
 
 // Joins the splits' records [T][H][n_splits][hd + 2] (output not yet divided, maximum, sum) into
-// the bf16 output [T][H][hd]; the prefill kernel's splits leave the same records.
+// the bf16 output [T][H][hd], hd the values' width.
 int sp_attn_combine(const float* part, void* out, int T, int H, int hd, int n_splits, hipStream_t st) {
-    SP_REQUIRE(T >= 0 && H > 0 && H <= 65535 && n_splits >= 1 && n_splits <= 256 && (hd == 64 || hd == 128),
+    SP_REQUIRE(T >= 0 && H > 0 && H <= 65535 && n_splits >= 1 && n_splits <= 256 && (hd == 32 || hd == 64 || hd == 128),
                "attn_combine: T=%d H=%d hd=%d splits=%d", T, H, hd, n_splits);
     if (T == 0) return 0;
     if (hd == 128) attn_decode_combine_kernel<128><<<dim3(T, H), 128, 0, st>>>(part, (bf16*)out, H, n_splits);
-    else attn_decode_combine_kernel<64><<<dim3(T, H), 64, 0, st>>>(part, (bf16*)out, H, n_splits);
+    else if (hd == 64) attn_decode_combine_kernel<64><<<dim3(T, H), 64, 0, st>>>(part, (bf16*)out, H, n_splits);
+    else attn_decode_combine_kernel<32><<<dim3(T, H), 64, 0, st>>>(part, (bf16*)out, H, n_splits);
     SP_LAUNCH_CHECK("attn_combine");
     return 0;
 }
 
-// Bytes of fp32 scratch that a call needs.
+// Bytes of fp32 scratch that a call needs (hd: the values' width).
 extern "C" size_t spite_attn_decode_workspace(int T, int H, int hd, int n_splits) {
     return (size_t)T * H * n_splits * (hd + 2) * sizeof(float);
 }
 
+// `v_dim`: width of the values (0: the keys' `hd`); the pairs (64, 32), (64, 64), (128, 64) and (128, 128) exist.
+// `keep`: with a chunk or a window the request's first so many keys are read as well.  `dist_bias` (device, fp32
+// [H][n_dist], or null): dist_bias[head][min(p - j, n_dist - 1)] is added to the scaled scores (before a cap).
 extern "C" int spite_attn_decode(const void* q, const void* k_pages, const void* v_pages, void* out, void* workspace,
                                  const int* positions, const int* seq_of_token, const int* block_table,
                                  int max_blocks, int T, int H, int G, int hd, int page_size, int vis, int span,
                                  float scale, float softcap, const float* slopes, int n_splits, int value_heads,
-                                 const float* sinks, hipStream_t st) {
+                                 const float* sinks, int v_dim, int keep, const float* dist_bias, int n_dist, hipStream_t st) {
     SP_REQUIRE(softcap >= 0.f && scale > 0.f, "attn_decode: scale %g, score cap %g", scale, softcap);
-    // value pages [pages][value_heads][hd][page]: kv head g reads value head g % value_heads (0: as many as kv heads)
+    // value pages [pages][value_heads][v_dim][page]: kv head g reads value head g % value_heads (0: as many as kv heads)
     if (value_heads <= 0) value_heads = G;
+    if (v_dim <= 0) v_dim = hd;
     SP_REQUIRE(G % value_heads == 0, "attn_decode: %d key heads over %d value heads", G, value_heads);
     SP_REQUIRE(T >= 0 && H > 0 && G > 0 && H % G == 0, "attn_decode: %d query heads over %d kv heads", H, G);
     SP_REQUIRE(H / G <= 16, "attn_decode: %d query heads per kv head, at most 16", H / G);
-    SP_REQUIRE(hd == 64 || hd == 128, "attn_decode: head size %d (this kernel has 64 and 128)", hd);
+    SP_REQUIRE((hd == 64 && (v_dim == 32 || v_dim == 64)) || (hd == 128 && (v_dim == 64 || v_dim == 128)),
+               "attn_decode: keys of %d with values of %d (this kernel has 64 / 32, 64 / 64, 128 / 64 and 128 / 128)", hd, v_dim);
     SP_REQUIRE(page_size > 0 && page_size % 32 == 0, "attn_decode: page size %d must be a multiple of 32", page_size);
     SP_REQUIRE(max_blocks > 0 && n_splits >= 1 && n_splits <= 256, "attn_decode: bad table width, or %d splits (at most 256)", n_splits);
     SP_REQUIRE(vis >= 0 && vis < SP_VIS_COUNT && (!sp_vis_has_span(vis) || span > 0), "attn_decode: chunk or window of %d", span);
+    SP_REQUIRE(keep >= 0 && (!dist_bias || n_dist > 0), "attn_decode: %d keys kept, distance bias of %d", keep, n_dist);
     SP_REQUIRE(G <= 65535 && T <= 65535, "attn_decode: too many heads or tokens for one launch");
     if (T == 0) return 0;
+    if (!sp_vis_has_span(vis)) keep = 0;
     const float sl = scale * 1.4426950408889634f, cr = softcap > 0.f ? scale / softcap : 0.f;
     dim3 grid(n_splits, G, T);
-    const size_t sh = (size_t)4 * 16 * (hd + 2) * sizeof(float);
-    if (hd == 128) {
-        attn_decode_kernel<128><<<grid, 256, sh, st>>>((const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages,
-            (float*)workspace, (bf16*)out, positions, seq_of_token, block_table, max_blocks, H, G, page_size, vis, span, sl, cr, n_splits, slopes, 1.0f / scale, value_heads, sinks);
-        SP_LAUNCH_CHECK("attn_decode");
-        if (n_splits > 1)
-            attn_decode_combine_kernel<128><<<dim3(T, H), 128, 0, st>>>((const float*)workspace, (bf16*)out, H, n_splits);
-    } else {
-        attn_decode_kernel<64><<<grid, 256, sh, st>>>((const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages,
-            (float*)workspace, (bf16*)out, positions, seq_of_token, block_table, max_blocks, H, G, page_size, vis, span, sl, cr, n_splits, slopes, 1.0f / scale, value_heads, sinks);
-        SP_LAUNCH_CHECK("attn_decode");
-        if (n_splits > 1)
-            attn_decode_combine_kernel<64><<<dim3(T, H), 64, 0, st>>>((const float*)workspace, (bf16*)out, H, n_splits);
-    }
-    SP_LAUNCH_CHECK("attn_decode_combine");
-    return 0;
+    const size_t sh = (size_t)4 * 16 * (v_dim + 2) * sizeof(float);
+#define SP_AD(HDV, VDV) do { \
+        auto kern = dist_bias ? attn_decode_kernel<HDV, VDV, true> : attn_decode_kernel<HDV, VDV, false>; \
+        kern<<<grid, 256, sh, st>>>((const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, (float*)workspace, (bf16*)out, positions, \
+            seq_of_token, block_table, max_blocks, H, G, page_size, vis, span, sl, cr, n_splits, slopes, 1.0f / scale, value_heads, sinks, \
+            keep, dist_bias, n_dist); } while (0)
+    if (hd == 128) { if (v_dim == 128) SP_AD(128, 128); else SP_AD(128, 64); }
+    else { if (v_dim == 64) SP_AD(64, 64); else SP_AD(64, 32); }
+#undef SP_AD
+    SP_LAUNCH_CHECK("attn_decode");
+    return n_splits > 1 ? sp_attn_combine((const float*)workspace, out, T, H, v_dim, n_splits, st) : 0;
 }
 
 // ---- the same call for callers that cannot allocate: the partial results go to an array of
@@ -316,5 +331,5 @@ extern "C" int spite_attn_decode_static(const void* q, const void* k_pages, cons
     SP_REQUIRE(e == hipSuccess && ptr != nullptr, "attn_decode_static: no address for the scratch array: %s",
                hipGetErrorString(e));
     return spite_attn_decode(q, k_pages, v_pages, out, ptr, positions, seq_of_token, block_table, max_blocks, T, H, G,
-                             hd, page_size, vis, span, scale, 0.f, nullptr, n_splits, 0, nullptr, st);
+                             hd, page_size, vis, span, scale, 0.f, nullptr, n_splits, 0, nullptr, hd, 0, nullptr, 0, st);
 }

@@ -23,7 +23,15 @@
 //     applied per element, values that the request does not own are taken as zero;
 //   * runs that no column of the wave reads: skipped.
 // Optional per-head slopes (a score bias slope * (key - query position)) and a smooth cap on
-// the scores take the per-element path in an instantiation of their own.
+// the scores take the per-element path in an instantiation of their own.  A bias by distance from a
+// table (one number for every distance from the table's end on) has a third: runs within the table's
+// reach take the per-element path, with the tables of the kv head's query heads in LDS where they fit;
+// runs beyond it are whole runs whose scores all get the column's last table entry, in the exponent's fma.
+//
+// Kept keys.  With a chunk or a window the first `keep` keys of the request may stay in sight: their
+// steps come before the rule's own, as edge steps.
+//
+// Keys and values may differ in width (HD and VD).
 //
 // Splits.  When the tiles are too few to fill the chip, or fill it unevenly (a long context
 // behind a short portion: every tile walks the same many keys, and 328 tiles on 256 compute
@@ -48,8 +56,10 @@
 #define PF_KEYS 128        // keys per step
 #define PF_RUNS (PF_KEYS / 32)
 
-// EXTRA: score slopes or a cap are in use (every run takes the per-element path)
-template <int HD, bool EXTRA>
+enum { PF_PLAIN = 0, PF_EXTRA = 1, PF_DIST = 2 };
+// MODE: PF_EXTRA, score slopes or a cap are in use (every run takes the per-element path); PF_DIST, a
+// bias by distance
+template <int HD, int VD, int MODE>
 __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2)))
 void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_pages,
                          const bf16* __restrict__ v_pages, bf16* __restrict__ out, float* __restrict__ part,
@@ -57,16 +67,18 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                          const int* __restrict__ block_table, int max_blocks, int tile_q,
                          int H, int G, int ps, int vis, int span, float scale_log2e, float cap_ratio,
                          const float* __restrict__ slopes, float inv_scale, int n_splits, int Gv,
-                         const float* __restrict__ sinks) {
+                         const float* __restrict__ sinks, int keep, const float* __restrict__ dist_bias, int n_dist,
+                         int tab_ld) {
+    constexpr bool EXTRA = MODE == PF_EXTRA, DIST = MODE == PF_DIST;
     constexpr int NS = HD / 16;                      // steps of 16 head elements in the score product
-    constexpr int NDT = HD / 32;                     // 32-row tiles of the output
+    constexpr int NDT = VD / 32;                     // 32-row tiles of the output
     constexpr int NC = HD / 32;                      // chunks of a K tile row
-    constexpr int TPR = HD / 16;                     // one-kilobyte tiles of a 32-key run (keys, or values)
-    constexpr int RUN = 32 * HD;                     // elements of a run
-    constexpr int STEP = PF_KEYS * HD;               // elements of the K (or V^T) tiles of one step
+    constexpr int RUN = 32 * HD, VRUN = 32 * VD;     // elements of a 32-key run of keys and of values
+    constexpr int STEP = PF_KEYS * HD, VSTEP = PF_KEYS * VD;    // elements of the K and of the V^T tiles of one step
     extern __shared__ __attribute__((aligned(16))) bf16 sm[];
-    bf16* Ks = sm;                                   // [2 buffers][PF_RUNS runs][TPR tiles][512]
-    bf16* Vs = sm + 2 * STEP;                        // the same for V^T
+    bf16* Ks = sm;                                   // [2 buffers][PF_RUNS runs][HD/16 tiles][512]
+    bf16* Vs = sm + 2 * STEP;                        // [2 buffers][PF_RUNS runs][VD/16 tiles][512]
+    float* tab_sh = (float*)(Vs + 2 * VSTEP);        // [H/G][tab_ld]: the distance tables, where tab_ld > 0
 
     // (the wave's number is the same in all of its lanes: saying so keeps what follows from it in scalar registers)
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -99,6 +111,13 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     const int pq = live ? positions[tok] : -1;
     const int lo = live ? sp_first_visible(pq, vis, span) : 0;
     const float slope = (EXTRA && slopes && live) ? slopes[head] * inv_scale : 0.f;
+    // a bias by distance: this column's table (in LDS, or where it lies in memory) and its last entry, in the exponent's units
+    const float* tab = DIST ? dist_bias + (size_t)(live ? head : 0) * n_dist : nullptr;
+    const int tab_at = DIST ? (live ? col % QH : 0) * tab_ld : 0;
+    const int reach = DIST ? n_dist - 1 : 0;         // every key at least this far away gets the last entry
+    const float far_l2e = DIST ? tab[reach] * 1.4426950408889634f : 0.f;
+    if (DIST && tab_ld > 0)
+        for (int i = tid; i < QH * n_dist; i += 512) tab_sh[(i / n_dist) * tab_ld + i % n_dist] = dist_bias[(size_t)g * QH * n_dist + i];
     bf16x8 qf[NS];
     {
         const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -131,10 +150,16 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     auto page_of = [&](int key) { const int i = key / ps; return i < max_blocks ? bt[i] : -1; };
 
     // ---- staging: every wave sends its share of the step's tiles from the pages into LDS.  A
-    // step has PF_RUNS runs of keys and as many of values, each TPR tiles of one kilobyte that
+    // step has PF_RUNS runs of keys and as many of values, each HD/16 or VD/16 tiles of one kilobyte that
     // lie in a row in its page; a wave sends one run's keys or values, a tile a load (16 bytes a lane).
     static_assert(PF_RUNS == 4, "eight waves send four runs of keys and four of values");
     const int hx = wave >> 1, is_v = wave & 1;
+    auto send = [&](const bf16* src, bf16* dst, auto tiles) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < decltype(tiles)::value; ++i)
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + i * 512 + lane * 8),
+                                             (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
+    };
     auto stage = [&](int u, int buf) __attribute__((always_inline)) {
         const int key = u * PF_KEYS + hx * 32;
         int pg = page_of(key);
@@ -142,13 +167,9 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         // values taken as zero
         pg = pg < 0 ? 0 : pg;
         // (value heads may be fewer than key heads: key head g reads value head g % Gv)
-        const size_t at = (is_v ? (size_t)pg * Gv + g % Gv : (size_t)pg * G + g) * (size_t)ps * HD + (size_t)((key % ps) >> 5) * RUN + lane * 8;
-        const bf16* src = (is_v ? v_pages : k_pages) + at;
-        bf16* dst = (is_v ? Vs : Ks) + buf * STEP + hx * RUN;
-#pragma unroll
-        for (int i = 0; i < TPR; ++i)
-            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + i * 512),
-                                             (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
+        const int blk = (key % ps) >> 5;
+        if (is_v) send(v_pages + ((size_t)pg * Gv + g % Gv) * (size_t)ps * VD + (size_t)blk * VRUN, Vs + buf * VSTEP + hx * VRUN, std::integral_constant<int, VD / 16>{});
+        else send(k_pages + ((size_t)pg * G + g) * (size_t)ps * HD + (size_t)blk * RUN, Ks + buf * STEP + hx * RUN, std::integral_constant<int, HD / 16>{});
     };
 
     // this lane's part of the operand addresses: row r of tile tt, the lane's half of the k run
@@ -156,12 +177,12 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     const int k_lane = tt * NC * 512 + hh * 128 + r * 8;
     const int v_lane = tt * 512 + hh * 128 + r * 8;
 
-    // ---- one run (32 keys, from key0) out of LDS, its tiles `at` elements into the buffers.
+    // ---- one run (32 keys, from key0) out of LDS, run h of buffer `buf`.
     // MASKED: tests per element.
-    auto run32 = [&](int key0, int at, auto masked_tag) __attribute__((always_inline)) {
+    auto run32 = [&](int key0, int buf, int h, auto masked_tag) __attribute__((always_inline)) {
         constexpr bool MASKED = decltype(masked_tag)::value;
-        const bf16* kb_ = Ks + at + k_lane;
-        const bf16* vb_ = Vs + at + v_lane;
+        const bf16* kb_ = Ks + buf * STEP + h * RUN + k_lane;
+        const bf16* vb_ = Vs + buf * VSTEP + h * VRUN + v_lane;
         f32x16 s;
 #pragma unroll
         for (int i = 0; i < 16; ++i) s[i] = 0.f;
@@ -206,7 +227,11 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                         // the raw score is replaced by the one that the scale turns into the capped score
                         if (cap_ratio > 0.f) v = tanhf(v * cap_ratio) / cap_ratio;
                     }
-                    const bool ok = key >= lo && key <= pq;
+                    if (DIST) {
+                        const int d = min(max(pq - key, 0), reach);
+                        v += (tab_ld > 0 ? tab_sh[tab_at + d] : tab[d]) * inv_scale;
+                    }
+                    const bool ok = sp_visible(key, pq, lo, keep);
                     s[4 * j + i] = ok ? (absent ? NAN : v) : -INFINITY;
                 }
         }
@@ -218,17 +243,20 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
             const auto sw = __builtin_amdgcn_permlane32_swap(__float_as_uint(mx), __float_as_uint(mx), false, false);
             mx = fmaxf(__uint_as_float(sw[0]), __uint_as_float(sw[1]));
         }
-        const float m_new = fmaxf(m_run, mx * scale_log2e);
+        // (a run out of the distance table's reach: all of its scores get the last entry)
+        const float c0 = DIST && !MASKED ? far_l2e : 0.f;
+        const float m_new = fmaxf(m_run, DIST ? fmaf(mx, scale_log2e, c0) : mx * scale_log2e);
         // a column with nothing visible so far keeps m = -inf: its weights are zero, not NaN
         const float m_safe = (MASKED && m_new == -INFINITY) ? 0.f : m_new;
         const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
+        const float m_off = DIST ? c0 - m_safe : -m_safe;
         float sum = 0.f;
         bf16x8 pf[2];                                // P, as the second product's B operands
 #pragma unroll
         for (int j = 0; j < 4; ++j)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                const float e = __builtin_amdgcn_exp2f(fmaf(s[4 * j + i], scale_log2e, -m_safe));
+                const float e = __builtin_amdgcn_exp2f(fmaf(s[4 * j + i], scale_log2e, m_off));
                 sum += e;
                 pf[j & 1][(j >> 1) * 4 + i] = (bf16)e;
             }
@@ -273,10 +301,10 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     auto edge_step = [&](int u, int buf) __attribute__((always_inline)) {
         for (int h = 0; h < PF_RUNS; ++h) {
             const int key0 = u * PF_KEYS + h * 32;
-            if (key0 > pq_max || key0 + 31 < lo_min) continue;            // nothing here for this wave
-            const bool whole = !EXTRA && key0 >= lo_max && key0 + 31 <= pq_min && page_of(key0) >= 0;
-            if (whole) run32(key0, buf * STEP + h * RUN, std::false_type{});
-            else run32(key0, buf * STEP + h * RUN, std::true_type{});
+            if (key0 > pq_max || (key0 + 31 < lo_min && key0 >= keep)) continue;            // nothing here for this wave
+            const bool whole = !EXTRA && (key0 >= lo_max || key0 + 31 < keep) && key0 + 31 <= pq_min - reach && page_of(key0) >= 0;
+            if (whole) run32(key0, buf, h, std::false_type{});
+            else run32(key0, buf, h, std::true_type{});
         }
     };
 
@@ -286,15 +314,19 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     // so the edges come first, in a loop whose waves choose their path run by run, and the
     // whole steps after them in a loop that holds the cheap path and nothing else (one loop with
     // both paths makes the compiler merge their ends, at the price of moving the operands of
-    // either into common registers in every run).  A split takes its share of that order.
+    // either into common registers in every run).  The kept keys' steps come before all others.  A split
+    // takes its share of that order.
+    const int n_keep = min((keep + PF_KEYS - 1) / PF_KEYS, u_first);
     int uA = u_last + 1, uB = u_last + 1;
     if (!EXTRA) {
         uA = max(u_first, (sp_first_visible(p_last, vis, span) + PF_KEYS - 1) / PF_KEYS);
-        uB = min(u_last + 1, (p_first + 1) / PF_KEYS);
+        uB = min(u_last + 1, max(p_first + 1 - reach, 0) / PF_KEYS);
         if (uA >= uB) uA = uB = u_last + 1;
     }
-    const int n_steps = u_last + 1 - u_first, n_low = uA - u_first, n_edge = n_steps - (uB - uA);
-    auto step_at = [&](int i) { return i < n_low ? u_first + i : (i < n_edge ? uB + (i - n_low) : uA + (i - n_edge)); };
+    const int n_steps = n_keep + u_last + 1 - u_first, n_low = n_keep + uA - u_first, n_edge = n_steps - (uB - uA);
+    auto step_at = [&](int i) {
+        return i < n_keep ? i : (i < n_low ? u_first + (i - n_keep) : (i < n_edge ? uB + (i - n_low) : uA + (i - n_edge)));
+    };
     const int i_begin = (int)((long)n_steps * split / n_splits), i_end = (int)((long)n_steps * (split + 1) / n_splits);
     bool poison = false;          // a whole step met a page that is not there
     if (i_begin < i_end) {
@@ -323,7 +355,7 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         if (i + 1 < i_end) stage(u + 1, buf ^ 1);
         if (pq_max >= 0) {
 #pragma unroll
-            for (int h = 0; h < PF_RUNS; ++h) run32(u * PF_KEYS + h * 32, buf * STEP + h * RUN, std::false_type{});
+            for (int h = 0; h < PF_RUNS; ++h) run32(u * PF_KEYS + h * 32, buf, h, std::false_type{});
         }
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
@@ -334,13 +366,13 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         const auto sw = __builtin_amdgcn_permlane32_swap(__float_as_uint(l_run), __float_as_uint(l_run), false, false);
         l_run = __uint_as_float(sw[0]) + __uint_as_float(sw[1]);
     }
-    // o[d][4j+i] of lane (n, hh): column n of the wave, head element 32d + 8j + 4hh + i
+    // o[d][4j+i] of lane (n, hh): column n of the wave, value element 32d + 8j + 4hh + i
     if (!live) return;
     if (n_splits > 1) {
         // This split's part of the tile, as it lies in the registers: a wave's stores are runs of
         // one kilobyte (a layout by columns would scatter them in pieces of 32 bytes).  The kernel
         // below reads it back the same way.
-        float* rec = part + ((size_t)blockIdx.x * 8 + wave) * (32 * HD + 64);
+        float* rec = part + ((size_t)blockIdx.x * 8 + wave) * (32 * VD + 64);
 #pragma unroll
         for (int d = 0; d < NDT; ++d)
 #pragma unroll
@@ -350,11 +382,11 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                 for (int i2 = 0; i2 < 4; ++i2) w[i2] = poison ? NAN : o[d][4 * j + i2];
                 *(f32x4*)(rec + ((d * 4 + j) * 64 + lane) * 4) = w;
             }
-        rec[32 * HD + lane] = hh == 0 ? m_run : (poison ? NAN : l_run);
+        rec[32 * VD + lane] = hh == 0 ? m_run : (poison ? NAN : l_run);
         return;
     }
     const float inv = poison ? NAN : 1.0f / fmaxf(l_run, 1e-30f);
-    bf16* orow = out + ((size_t)tok * H + head) * HD;
+    bf16* orow = out + ((size_t)tok * H + head) * VD;
 #pragma unroll
     for (int d = 0; d < NDT; ++d)
 #pragma unroll
@@ -369,7 +401,7 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
 // Joins the splits of every tile: workgroup (tile, kv head) reads the records that its splits'
 // workgroups left, in the registers' own layout, weighs them by their maxima and writes the
 // output as the unsplit kernel does.
-template <int HD>
+template <int HD>      // HD: the values' width
 __global__ __launch_bounds__(512)
 void attn_prefill_join_kernel(const float* __restrict__ part, bf16* __restrict__ out, const int* __restrict__ cu_seqlens,
                               int n_seqs, int tile_q, int H, int G, int n_splits) {
@@ -423,21 +455,34 @@ void attn_prefill_join_kernel(const float* __restrict__ part, bf16* __restrict__
         }
 }
 
-template <int HD, bool EXTRA>
+// LDS that a launch may use beside the buffers of keys and values for the distance tables.
+#define PF_TAB_BYTES (32 * 1024)
+
+template <int HD, int VD, int MODE>
 static int launch_prefill(const void* q, const void* k_pages, const void* v_pages, void* out, float* part, const int* positions,
                           const int* cu_seqlens, int n_seqs, const int* block_table, int max_blocks, int tile_q,
                           long n_tiles, int H, int G, int page_size, int vis, int span, float sl, float cr,
-                          const float* slopes, float inv_scale, int n_splits, int Gv, const float* sinks, hipStream_t st) {
-    const size_t sh = (size_t)2 * 2 * PF_KEYS * HD * sizeof(bf16);
+                          const float* slopes, float inv_scale, int n_splits, int Gv, const float* sinks, int keep,
+                          const float* dist_bias, int n_dist, hipStream_t st) {
+    const size_t base = (size_t)2 * PF_KEYS * (HD + VD) * sizeof(bf16);
+    size_t sh = base;
+    int tab_ld = 0;
+    if (MODE == PF_DIST) {
+        // a table row a head of the kv head, rows a part of the banks apart so that the heads of a wave's columns do not meet
+        const int qh = H / G, apart = qh <= 32 ? 32 / qh : 1;
+        const long ld = ((long)n_dist + 31) / 32 * 32 + apart;
+        if (ld * qh * (long)sizeof(float) <= PF_TAB_BYTES) { tab_ld = (int)ld; sh += (size_t)ld * qh * sizeof(float); }
+    }
     static bool allowed = false;          // one flag per instantiation: more LDS than the default limit
     if (!allowed) {
-        hipError_t e = hipFuncSetAttribute((const void*)attn_prefill_kernel<HD, EXTRA>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)sh);
-        SP_REQUIRE(e == hipSuccess, "attn_prefill: %zu bytes of LDS refused: %s", sh, hipGetErrorString(e));
+        const size_t most = base + (MODE == PF_DIST ? PF_TAB_BYTES : 0);
+        hipError_t e = hipFuncSetAttribute((const void*)attn_prefill_kernel<HD, VD, MODE>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)most);
+        SP_REQUIRE(e == hipSuccess, "attn_prefill: %zu bytes of LDS refused: %s", most, hipGetErrorString(e));
         allowed = true;
     }
-    attn_prefill_kernel<HD, EXTRA><<<dim3((unsigned)(n_tiles * G * n_splits)), 512, sh, st>>>((const bf16*)q, (const bf16*)k_pages,
+    attn_prefill_kernel<HD, VD, MODE><<<dim3((unsigned)(n_tiles * G * n_splits)), 512, sh, st>>>((const bf16*)q, (const bf16*)k_pages,
         (const bf16*)v_pages, (bf16*)out, part, positions, cu_seqlens, n_seqs, block_table, max_blocks, tile_q, H, G, page_size,
-        vis, span, sl, cr, slopes, inv_scale, n_splits, Gv, sinks);
+        vis, span, sl, cr, slopes, inv_scale, n_splits, Gv, sinks, keep, dist_bias, n_dist, tab_ld);
     SP_LAUNCH_CHECK("attn_prefill");
     return 0;
 }
@@ -474,23 +519,32 @@ extern "C" int spite_attn_prefill_splits(const int* counts, int n_seqs, int H, i
 // (spite_attn_prefill_workspace bytes) and are joined by a second kernel.  `slopes` (device,
 // fp32 [H], or null): a bias slopes[head] * (key position - query position) added to the scaled
 // scores before the cap.  `sinks` (device, fp32 [H], or null): one more term exp(sinks[head]) in the
-// denominator of every softmax of that head.
+// denominator of every softmax of that head.  `v_dim`: width of the values (0: the keys' `hd`); the pairs
+// (64, 32), (64, 64), (128, 64) and (128, 128) exist.  `keep`: with a chunk or a window the request's first so
+// many keys are read as well.  `dist_bias` (device, fp32 [H][n_dist], or null; not beside slopes or a cap):
+// dist_bias[head][min(p - j, n_dist - 1)] is added to the scaled scores.
 extern "C" int spite_attn_prefill(const void* q, const void* k_pages, const void* v_pages, void* out, void* workspace,
                                   const int* positions, const int* cu_seqlens, const int* counts, int n_seqs,
                                   const int* block_table, int max_blocks, int H, int G, int hd, int page_size,
                                   int vis, int span, float scale, float softcap, const float* slopes, int n_splits,
-                                  int value_heads, const float* sinks, hipStream_t st) {
+                                  int value_heads, const float* sinks, int v_dim, int keep, const float* dist_bias, int n_dist,
+                                  hipStream_t st) {
     SP_REQUIRE(softcap >= 0.f && scale > 0.f, "attn_prefill: scale %g, score cap %g", scale, softcap);
-    // value pages [pages][value_heads][hd][page]: kv head g reads value head g % value_heads (0: as many as kv heads)
+    // value pages [pages][value_heads][v_dim][page]: kv head g reads value head g % value_heads (0: as many as kv heads)
     if (value_heads <= 0) value_heads = G;
+    if (v_dim <= 0) v_dim = hd;
     SP_REQUIRE(G % value_heads == 0, "attn_prefill: %d key heads over %d value heads", G, value_heads);
     SP_REQUIRE(n_seqs >= 0 && H > 0 && G > 0 && H % G == 0, "attn_prefill: %d query heads over %d kv heads", H, G);
     SP_REQUIRE(H / G <= PF_COLS, "attn_prefill: %d query heads per kv head, at most %d", H / G, PF_COLS);
-    SP_REQUIRE(hd == 64 || hd == 128, "attn_prefill: head size %d (this kernel has 64 and 128)", hd);
+    SP_REQUIRE((hd == 64 && (v_dim == 32 || v_dim == 64)) || (hd == 128 && (v_dim == 64 || v_dim == 128)),
+               "attn_prefill: keys of %d with values of %d (this kernel has 64 / 32, 64 / 64, 128 / 64 and 128 / 128)", hd, v_dim);
     SP_REQUIRE(page_size > 0 && page_size % 32 == 0, "attn_prefill: page size %d must be a multiple of 32", page_size);
     SP_REQUIRE(max_blocks > 0, "attn_prefill: bad table width");
     SP_REQUIRE(vis >= 0 && vis < SP_VIS_COUNT && (!sp_vis_has_span(vis) || span > 0), "attn_prefill: chunk or window of %d", span);
     SP_REQUIRE(n_splits >= 1 && n_splits <= 256 && (n_splits == 1 || workspace), "attn_prefill: %d splits (1 to 256; more than one need a workspace)", n_splits);
+    SP_REQUIRE(keep >= 0 && (!dist_bias || n_dist > 0), "attn_prefill: %d keys kept, distance bias of %d", keep, n_dist);
+    SP_REQUIRE(!dist_bias || (!slopes && softcap == 0.f), "attn_prefill: a bias by distance goes with neither slopes nor a cap");
+    if (!sp_vis_has_span(vis)) keep = 0;
     long T = 0;
     for (int s = 0; s < n_seqs; ++s) {
         SP_REQUIRE(counts[s] >= 0, "attn_prefill: request %d with %d tokens", s, counts[s]);
@@ -501,23 +555,26 @@ extern "C" int spite_attn_prefill(const void* q, const void* k_pages, const void
     if (tiles == 0) return 0;
     SP_REQUIRE(tiles * G * n_splits <= 0x7fffffffL && T <= 0x7fffffffL, "attn_prefill: too many tiles");
     const float sl = scale * 1.4426950408889634f, cr = softcap > 0.f ? scale / softcap : 0.f;
-    const bool extra = cr > 0.f || slopes != nullptr;
-#define SP_PF(HDV, EX) launch_prefill<HDV, EX>(q, k_pages, v_pages, out, (float*)workspace, positions, cu_seqlens, n_seqs, \
-        block_table, max_blocks, tile_q, tiles, H, G, page_size, vis, span, sl, cr, slopes, 1.0f / scale, n_splits, value_heads, sinks, st)
-    const int rc = hd == 128 ? (extra ? SP_PF(128, true) : SP_PF(128, false)) : (extra ? SP_PF(64, true) : SP_PF(64, false));
+    const int mode = dist_bias ? PF_DIST : (cr > 0.f || slopes ? PF_EXTRA : PF_PLAIN);
+#define SP_PF(HDV, VDV, MD) launch_prefill<HDV, VDV, MD>(q, k_pages, v_pages, out, (float*)workspace, positions, cu_seqlens, n_seqs, \
+        block_table, max_blocks, tile_q, tiles, H, G, page_size, vis, span, sl, cr, slopes, 1.0f / scale, n_splits, value_heads, sinks, \
+        keep, dist_bias, n_dist, st)
+#define SP_PFM(HDV, VDV) (mode == PF_DIST ? SP_PF(HDV, VDV, PF_DIST) : (mode == PF_EXTRA ? SP_PF(HDV, VDV, PF_EXTRA) : SP_PF(HDV, VDV, PF_PLAIN)))
+    const int rc = hd == 128 ? (v_dim == 128 ? SP_PFM(128, 128) : SP_PFM(128, 64)) : (v_dim == 64 ? SP_PFM(64, 64) : SP_PFM(64, 32));
+#undef SP_PFM
 #undef SP_PF
     if (rc != 0 || n_splits == 1) return rc;
-    if (hd == 128)
-        attn_prefill_join_kernel<128><<<dim3((unsigned)(tiles * G)), 512, 0, st>>>((const float*)workspace, (bf16*)out, cu_seqlens,
-                                                                                  n_seqs, tile_q, H, G, n_splits);
-    else
-        attn_prefill_join_kernel<64><<<dim3((unsigned)(tiles * G)), 512, 0, st>>>((const float*)workspace, (bf16*)out, cu_seqlens,
-                                                                                 n_seqs, tile_q, H, G, n_splits);
+#define SP_PJ(VDV) attn_prefill_join_kernel<VDV><<<dim3((unsigned)(tiles * G)), 512, 0, st>>>((const float*)workspace, (bf16*)out, cu_seqlens, \
+        n_seqs, tile_q, H, G, n_splits)
+    if (v_dim == 128) SP_PJ(128);
+    else if (v_dim == 64) SP_PJ(64);
+    else SP_PJ(32);
+#undef SP_PJ
     SP_LAUNCH_CHECK("attn_prefill_join");
     return 0;
 }
 
-// Bytes of fp32 scratch that a call with `n_splits` > 1 needs: one record of 256 columns per
+// Bytes of fp32 scratch that a call with `n_splits` > 1 needs (hd: the values' width): one record of 256 columns per
 // tile, kv head and split.
 extern "C" size_t spite_attn_prefill_workspace(const int* counts, int n_seqs, int H, int G, int hd, int n_splits) {
     if (n_splits <= 1 || n_seqs <= 0 || H <= 0 || G <= 0 || H % G || H / G > PF_COLS) return 0;

@@ -28,7 +28,9 @@
 // values turn by pos * inv_freq_v[m] in pairs (m, m + Vd/2).  Keys go to [page][GK][offset][Dp],
 // values to [page][GV][Vd][offset] (or the operand order of common.h).  Dp >= D is the width that
 // queries and keys are stored with: the elements behind D are written as zeros (a head narrower than
-// what an attention kernel takes is widened this way; zeros add nothing to a score).
+// what an attention kernel takes is widened this way; zeros add nothing to a score).  With `v_other` (rows
+// `ld_other` apart) the values are blended with another layer's of the same token before they are cached:
+// (1 - v_lam) v + v_lam other.
 template <typename T>
 __global__ __launch_bounds__(WIDE_NT)
 void qkv_prepare_kernel(const T* __restrict__ qkv, int ld, const float* __restrict__ bias,
@@ -37,7 +39,8 @@ void qkv_prepare_kernel(const T* __restrict__ qkv, int ld, const float* __restri
                         const int* __restrict__ positions, const int* __restrict__ slot_map,
                         const float* __restrict__ inv_freq, int rot, float rot_mag, const float* __restrict__ inv_freq_v,
                         int HQ, int GK, int GV, int D, int Vd, int ps, int k_tiled, int v_tiled, int Dp, int hpb,
-                        int head_norm, float qt_coef, int qt_every, int v_from_k) {
+                        int head_norm, float qt_coef, int qt_every, int v_from_k,
+                        const T* __restrict__ v_other, int ld_other, float v_lam) {
     extern __shared__ float sm[];
     __shared__ float red[WIDE_NT / 64];
     const int rh = rot >> 1, vh = inv_freq_v ? (Vd >> 1) : 0;
@@ -127,7 +130,10 @@ void qkv_prepare_kernel(const T* __restrict__ qkv, int ld, const float* __restri
     for (int it = tid; it < (v_hi > v_lo ? v_hi - v_lo : 0) * vitems; it += WIDE_NT) {
         const int g = v_lo + it / vitems, i = it % vitems;
         T* slab = v_pages + (page * GV + g) * (size_t)Vd * ps;
-        auto load = [&](int c) { return to_f32<T>(row[vbase + g * Vd + c]) + (bias ? bias[vbase + g * Vd + c] : 0.f); };
+        auto load = [&](int c) {
+            const float v = to_f32<T>(row[vbase + g * Vd + c]) + (bias ? bias[vbase + g * Vd + c] : 0.f);
+            return v_other ? (1.0f - v_lam) * v + v_lam * to_f32<T>(v_other[(size_t)t * ld_other + g * Vd + c]) : v;
+        };
         if (i < vh) {
             const float a = load(i), b = load(i + vh);
             slab[sp_v_index(i, off, Vd, ps, v_tiled)] = from_f32<T>(a * csv[i] - b * snv[i]);
@@ -150,7 +156,8 @@ void qkv_prepare_vec_kernel(const bf16* __restrict__ qkv, int ld, const float* _
                             const int* __restrict__ positions, const int* __restrict__ slot_map,
                             const float* __restrict__ inv_freq, int rot, float rot_mag, const float* __restrict__ inv_freq_v,
                             int HQ, int GK, int GV, int D, int Vd, int ps, int k_tiled, int v_tiled, int Dp, int hpb,
-                            int head_norm, float qt_coef, int qt_every, int v_from_k) {
+                            int head_norm, float qt_coef, int qt_every, int v_from_k,
+                            const bf16* __restrict__ v_other, int ld_other, float v_lam) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ float red[WIDE_NT / 64];
     const int rh = rot >> 1, vh = inv_freq_v ? (Vd >> 1) : 0;
@@ -237,7 +244,10 @@ void qkv_prepare_vec_kernel(const bf16* __restrict__ qkv, int ld, const float* _
     for (int it = tid; it < (v_hi > v_lo ? v_hi - v_lo : 0) * vitems; it += WIDE_NT) {
         const int g = v_lo + it / vitems, i = it % vitems;
         bf16* slab = v_pages + (page * GV + g) * (size_t)Vd * ps;
-        auto load = [&](int c) { return (float)row[vbase + g * Vd + c] + (bias ? bias[vbase + g * Vd + c] : 0.f); };
+        auto load = [&](int c) {
+            const float v = (float)row[vbase + g * Vd + c] + (bias ? bias[vbase + g * Vd + c] : 0.f);
+            return v_other ? (1.0f - v_lam) * v + v_lam * (float)v_other[(size_t)t * ld_other + g * Vd + c] : v;
+        };
         if (i < vh) {
             const float a = load(i), b = load(i + vh);
             slab[sp_v_index(i, off, Vd, ps, v_tiled)] = (bf16)(a * csv[i] - b * snv[i]);
@@ -253,12 +263,14 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
                                  float eps, void* q_out, void* k_pages, void* v_pages, const int* positions,
                                  const int* slot_map, const float* inv_freq, int rot, float rot_mag, const float* inv_freq_v,
                                  int T, int HQ, int GK, int GV, int D, int Vd, int page_size, int k_tiled, int v_tiled,
-                                 int Dp, int head_norm, float qt_coef, int qt_every, int v_from_k, hipStream_t st) {
+                                 int Dp, int head_norm, float qt_coef, int qt_every, int v_from_k,
+                                 const void* v_other, int ld_other, float v_lam, hipStream_t st) {
     if (Dp <= 0) Dp = D;
     SP_REQUIRE(Dp >= D, "qkv_prepare: heads of %d stored with %d elements", D, Dp);
     SP_REQUIRE(T >= 0 && HQ > 0 && GK > 0 && GV > 0 && D > 0 && Vd > 0 && page_size > 0, "qkv_prepare: bad sizes");
     SP_REQUIRE(ld >= (HQ + GK) * D + (v_from_k ? 0 : GV * Vd), "qkv_prepare: rows of %d elements for %d", ld, (HQ + GK) * D + (v_from_k ? 0 : GV * Vd));
     SP_REQUIRE(!v_from_k || (GV == GK && Vd == D && !inv_freq_v), "qkv_prepare: values taken from the keys have the keys' heads and width");
+    SP_REQUIRE(!v_other || ld_other >= GV * Vd, "qkv_prepare: rows of %d values to blend with, %d wanted", ld_other, GV * Vd);
     SP_REQUIRE(!head_norm || (wq && wk), "qkv_prepare: a head norm needs its two weight vectors");
     SP_REQUIRE(qt_every >= 0, "qkv_prepare: query temperature every %d positions", qt_every);
     SP_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= D, "qkv_prepare: %d turning elements of a head of %d", rot, D);
@@ -283,16 +295,19 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
         && al(bias, 16) && al(wq, 16) && al(wk, 16)) {
         // (the sine and cosine tables are read four at a time: the second starts rot/2 floats behind the first)
         qkv_prepare_vec_kernel<<<grid, WIDE_NT, sh, st>>>((const bf16*)qkv, ld, bias, wq, wk, eps, (bf16*)q_out, (bf16*)k_pages,
-            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k);
+            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k,
+            (const bf16*)v_other, ld_other, v_lam);
         SP_LAUNCH_CHECK("qkv_prepare");
         return 0;
     }
     if (dtype == SP_F32)
         qkv_prepare_kernel<float><<<grid, WIDE_NT, sh, st>>>((const float*)qkv, ld, bias, wq, wk, eps, (float*)q_out, (float*)k_pages,
-            (float*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k);
+            (float*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k,
+            (const float*)v_other, ld_other, v_lam);
     else if (dtype == SP_BF16)
         qkv_prepare_kernel<bf16><<<grid, WIDE_NT, sh, st>>>((const bf16*)qkv, ld, bias, wq, wk, eps, (bf16*)q_out, (bf16*)k_pages,
-            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k);
+            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k,
+            (const bf16*)v_other, ld_other, v_lam);
     else return sp_fail("qkv_prepare: unknown dtype %d", dtype);
     SP_LAUNCH_CHECK("qkv_prepare");
     return 0;
@@ -303,7 +318,9 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
 // visible key, so the order of every sum depends on the query's position alone: a token gives
 // the same bits whether it comes in a whole prompt, a portion or alone.  With `sinks` (fp32 [HQ])
 // every head's softmax has one more term in its denominator, exp(sinks[h]): a score that is not
-// scaled, belongs to no key and brings no value.
+// scaled, belongs to no key and brings no value.  With `dist_bias` (fp32 [HQ][n_dist]) the scaled score gets
+// dist_bias[h][min(p - j, n_dist - 1)] added.  With `keep` the request's first `keep` keys are read beside the
+// rule's (visibility.h): they are walked first, in tiles that start at key 0.
 #define WIDE_MAX_V 8   // value widths up to 512
 
 template <typename T, typename TO>
@@ -312,7 +329,8 @@ void attn_wide_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
                       TO* __restrict__ out, const int* __restrict__ positions,
                       const int* __restrict__ seq_of_token, const int* __restrict__ block_table,
                       int max_blocks, int HQ, int GK, int GV, int D, int Vd, int ps, int vis, int span, float scale,
-                      int k_tiled, int v_tiled, const float* __restrict__ sinks, const float* __restrict__ slopes) {
+                      int k_tiled, int v_tiled, const float* __restrict__ sinks, const float* __restrict__ slopes,
+                      int keep, const float* __restrict__ dist_bias, int n_dist) {
     extern __shared__ float smem[];
     float* q_sh = smem;                 // [D]
     float* p_sh = smem + D;             // [64]
@@ -333,11 +351,17 @@ void attn_wide_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
 #pragma unroll
     for (int u = 0; u < WIDE_MAX_V; ++u) o[u] = 0.f;
 
-    for (int j0 = lo; j0 <= p; j0 += 64) {
+    // two runs of keys: the kept ones below the rule's first, then the rule's own (one run where nothing lies between)
+    const int n_kept = keep < lo ? keep : 0;
+    const int first = keep < lo ? lo : 0 < keep ? 0 : lo;
+    const int kept_tiles = (n_kept + 63) >> 6, tiles = kept_tiles + (p - first) / 64 + 1;
+    for (int tile = 0; tile < tiles; ++tile) {
+        const int j0 = tile < kept_tiles ? tile * 64 : first + (tile - kept_tiles) * 64;
+        const int j_end = (tile < kept_tiles ? n_kept : p + 1) - j0;           // keys of this tile
         const int j = j0 + lane;
         float s = -INFINITY;
         int page = -1;
-        if (j <= p) {
+        if (lane < j_end) {
             page = bt[j / ps];
             if (page < 0) {
                 s = NAN;   // a page that was given back is asked for: poison the result
@@ -347,11 +371,12 @@ void attn_wide_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
                 for (int c = 0; c < D; ++c) acc = fmaf(q_sh[c], to_f32<T>(kr[sp_k_index(j % ps, c, D, k_tiled)]), acc);
                 s = acc * scale;
                 if (slopes) s += slopes[h] * (float)(j - p);       // a bias that grows with the distance
+                if (dist_bias) s += dist_bias[(size_t)h * n_dist + (p - j < n_dist ? p - j : n_dist - 1)];
             }
         }
         const float m_new = fmaxf(m, wave_max(s));
         const float alpha = expf(m - m_new);
-        const float pj = (j <= p) ? expf(s - m_new) : 0.f;
+        const float pj = lane < j_end ? expf(s - m_new) : 0.f;
         l = l * alpha + wave_sum(pj);
         m = m_new;
         __syncthreads();
@@ -359,7 +384,7 @@ void attn_wide_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
         page_sh[lane] = page;
         off_sh[lane] = j % ps;
         __syncthreads();
-        const int n_valid = (p - j0 + 1) < 64 ? (p - j0 + 1) : 64;
+        const int n_valid = j_end < 64 ? j_end : 64;
 #pragma unroll
         for (int u = 0; u < WIDE_MAX_V; ++u) {
             const int c = lane + u * 64;
@@ -386,7 +411,9 @@ void attn_wide_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
 extern "C" int spite_attn_wide(const void* q, const void* k_pages, const void* v_pages, void* out, int dtype, int out_dtype,
                                const int* positions, const int* seq_of_token, const int* block_table,
                                int max_blocks, int T, int HQ, int GK, int GV, int D, int Vd, int page_size, int vis, int span,
-                               float scale, int k_tiled, int v_tiled, const float* sinks, const float* slopes, hipStream_t st) {
+                               float scale, int k_tiled, int v_tiled, const float* sinks, const float* slopes,
+                               int keep, const float* dist_bias, int n_dist, hipStream_t st) {
+    SP_REQUIRE(keep >= 0 && (!dist_bias || n_dist > 0), "attention: %d keys kept, distance bias of %d", keep, n_dist);
     SP_REQUIRE(T >= 0 && HQ > 0 && GK > 0 && GV > 0 && HQ % GK == 0 && GK % GV == 0,
                "attention: %d query heads over %d key heads over %d value heads", HQ, GK, GV);
     SP_REQUIRE(D > 0 && D <= 4096 && Vd > 0 && Vd <= 64 * WIDE_MAX_V, "attention: keys of %d, values of %d (at most %d)", D, Vd, 64 * WIDE_MAX_V);
@@ -399,7 +426,8 @@ extern "C" int spite_attn_wide(const void* q, const void* k_pages, const void* v
     dim3 grid(T, HQ);
     const size_t sh = (size_t)(D + 64) * sizeof(float) + 128 * sizeof(int);
 #define SP_AW(TI, TO) attn_wide_kernel<TI, TO><<<grid, 64, sh, st>>>((const TI*)q, (const TI*)k_pages, (const TI*)v_pages, (TO*)out, \
-        positions, seq_of_token, block_table, max_blocks, HQ, GK, GV, D, Vd, page_size, vis, span, scale, k_tiled, v_tiled, sinks, slopes)
+        positions, seq_of_token, block_table, max_blocks, HQ, GK, GV, D, Vd, page_size, vis, span, scale, k_tiled, v_tiled, sinks, slopes, \
+        sp_vis_has_span(vis) ? keep : 0, dist_bias, n_dist)
     if (dtype == SP_F32 && out_dtype == SP_F32) SP_AW(float, float);
     else if (dtype == SP_BF16 && out_dtype == SP_BF16) SP_AW(bf16, bf16);
     else if (dtype == SP_BF16 && out_dtype == SP_F32) SP_AW(bf16, float);

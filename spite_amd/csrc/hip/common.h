@@ -151,7 +151,7 @@ __device__ __forceinline__ float wave_dot_row(const float* __restrict__ w, const
 // The gate's activation in a gated product act(gate) * up: SP_ACT_SILU g * sigmoid(g),
 // SP_ACT_GELU_TANH 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))), or SP_ACT_RELU max(g, 0).
 // `fast`: the short exponential (the bfloat16 products); the 32-bit path takes the accurate routines.
-enum { SP_ACT_NONE = 0, SP_ACT_SILU = 1, SP_ACT_GELU_TANH = 2, SP_ACT_RELU = 3 };
+enum { SP_ACT_NONE = 0, SP_ACT_SILU = 1, SP_ACT_GELU_TANH = 2, SP_ACT_RELU = 3, SP_ACT_CLAMPED = 4, SP_ACT_LAST = SP_ACT_CLAMPED };
 __device__ __forceinline__ float sp_gate_act(float g, int act, bool fast) {
     if (act == SP_ACT_RELU) return fmaxf(g, 0.f);
     if (act == SP_ACT_GELU_TANH) {
@@ -161,6 +161,20 @@ __device__ __forceinline__ float sp_gate_act(float g, int act, bool fast) {
         return 0.5f * g * (1.0f + t);
     }
     return g / (1.0f + (fast ? __expf(-g) : expf(-g)));
+}
+
+// The epilogue of a gated product: act(gate) * up, or, SP_ACT_CLAMPED, the form whose two halves are bounded:
+// g = min(gate, limit), u = up within [-limit, limit], g * sigmoid(1.702 g) * (u + 1).  (Comparisons, not
+// fmin / fmax: a NaN stays one.)
+#define SP_CLAMPED_SLOPE 1.702f
+__device__ __forceinline__ float sp_gated(float g, float u, int act, float limit, bool fast) {
+    if (act == SP_ACT_CLAMPED) {
+        g = g > limit ? limit : g;
+        u = u > limit ? limit : (u < -limit ? -limit : u);
+        const float z = -SP_CLAMPED_SLOPE * g;
+        return g / (1.0f + (fast ? __expf(z) : expf(z))) * (u + 1.0f);
+    }
+    return sp_gate_act(g, act, fast) * u;
 }
 
 // An activation on its own (no gate): SP_UNARY_GELU 0.5 z (1 + erf(z / sqrt 2)), SP_UNARY_GELU_TANH,

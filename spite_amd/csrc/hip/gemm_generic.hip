@@ -7,7 +7,7 @@
 // [offsets[g], offsets[g+1]) and multiplies them with W + g*w_group_stride.  A slot reads
 // row a_rows[s] of A (times a_scale[s], in fp32, before the product) and writes row
 // y_rows[s] of Y.  With `glu` the group's W holds 2N rows, gate rows first, and the kernel
-// writes act(gate) * up (`glu`: 1 silu, 2 the tanh form of gelu).
+// writes act(gate) * up (`glu`: the activation's code, `act_limit` its bound where it has one; see sp_gated).
 #include "common.h"
 
 #define GBM 64
@@ -20,7 +20,7 @@ void gemm_generic_kernel(const T* __restrict__ A, int lda, const T* __restrict__
                          TY* __restrict__ Y, int ldy, int M, int N, int K,
                          const int* __restrict__ offsets, int n_groups,
                          const int* __restrict__ a_rows, const float* __restrict__ a_scale,
-                         const int* __restrict__ y_rows, int act) {
+                         const int* __restrict__ y_rows, int act, float act_limit) {
     __shared__ float As[GBK][GBM + 1];
     __shared__ float Ws[GLU ? 2 : 1][GBK][GBN + 1];
     // ---- which group and which of its row tiles
@@ -88,7 +88,7 @@ void gemm_generic_kernel(const T* __restrict__ A, int lda, const T* __restrict__
             const int n = n0 + tn + j;
             if (n >= N) continue;
             float v = acc_g[i][j];
-            if (GLU) v = sp_gate_act(v, act, false) * acc_u[i][j];
+            if (GLU) v = sp_gated(v, acc_u[i][j], act, act_limit, false);
             Y[yr * ldy + n] = from_f32<TY>(v);
         }
     }
@@ -97,17 +97,18 @@ void gemm_generic_kernel(const T* __restrict__ A, int lda, const T* __restrict__
 extern "C" int spite_gemm_generic(const void* A, int lda, const void* W, long w_group_stride, int dtype,
                                   void* Y, int y_dtype, int ldy, int M, int N, int K,
                                   const int* offsets, int n_groups, const int* a_rows,
-                                  const float* a_scale, const int* y_rows, int glu, hipStream_t st) {
+                                  const float* a_scale, const int* y_rows, int glu, float act_limit, hipStream_t st) {
     SP_REQUIRE(M >= 0 && N > 0 && K > 0 && lda >= K && ldy >= N, "gemm: bad sizes M=%d N=%d K=%d lda=%d ldy=%d",
                M, N, K, lda, ldy);
     SP_REQUIRE(!offsets || n_groups > 0, "gemm: grouped call without groups");
+    SP_REQUIRE(glu >= 0 && glu <= SP_ACT_LAST && (glu != SP_ACT_CLAMPED || act_limit > 0.f), "gemm: activation code %d with bound %g", glu, act_limit);
     if (M == 0) return 0;
     // row tiles: a group with rows has 1 + (rows - 1) / tile of them, so groups with rows + M / tile bounds them
     const int m_tiles = offsets ? M / GBM + (n_groups < M ? n_groups : M) : (M + GBM - 1) / GBM;
     SP_REQUIRE(m_tiles <= 65535, "gemm: too many row tiles (%d)", m_tiles);
     dim3 grid((N + GBN - 1) / GBN, m_tiles);
 #define SP_GEMM_LAUNCH(T, TY, GLU) gemm_generic_kernel<T, TY, GLU><<<grid, 256, 0, st>>>( \
-        (const T*)A, lda, (const T*)W, w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu)
+        (const T*)A, lda, (const T*)W, w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu, act_limit)
     if (dtype == SP_F32 && y_dtype == SP_F32) { if (glu) SP_GEMM_LAUNCH(float, float, 1); else SP_GEMM_LAUNCH(float, float, 0); }
     else if (dtype == SP_BF16 && y_dtype == SP_BF16) { if (glu) SP_GEMM_LAUNCH(bf16, bf16, 1); else SP_GEMM_LAUNCH(bf16, bf16, 0); }
     else if (dtype == SP_BF16 && y_dtype == SP_F32) { if (glu) SP_GEMM_LAUNCH(bf16, float, 1); else SP_GEMM_LAUNCH(bf16, float, 0); }

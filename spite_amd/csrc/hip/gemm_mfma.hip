@@ -30,7 +30,7 @@ __global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2)))
 void gemm_mfma_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restrict__ W, long w_group_stride,
                       TY* __restrict__ Y, int ldy, int M, int N, int K,
                       const int* __restrict__ offsets, int n_groups, const int* __restrict__ a_rows,
-                      const float* __restrict__ a_scale, const int* __restrict__ y_rows, int m_tiles, int n_tiles, int act) {
+                      const float* __restrict__ a_scale, const int* __restrict__ y_rows, int m_tiles, int n_tiles, int act, float act_limit) {
     static_assert(WN * WM == 8, "eight waves");
     constexpr int BM = 128 * WM, BN = 64 * WN;
     constexpr int NCOLS = GLU ? BN / 2 : BN;        // output columns per workgroup
@@ -164,7 +164,7 @@ void gemm_mfma_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restric
                 for (int i = 0; i < 4; ++i) {
                     if (n + i < N) {
                         const float gv = acc[a][b][i] * sc, uv = acc[a + TG][b][i] * sc;
-                        yrow[n + i] = from_f32<TY>(sp_gate_act(gv, act, true) * uv);
+                        yrow[n + i] = from_f32<TY>(sp_gated(gv, uv, act, act_limit, true));
                     }
                 }
             }
@@ -183,7 +183,7 @@ void gemm_mfma_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restric
 template <int WN, int WM>
 static int launch_mfma(const void* X, int ldx, const void* W, long w_group_stride, void* Y, int y_dtype, int ldy, int M,
                        int N, int K, const int* offsets, int n_groups, const int* a_rows, const float* a_scale,
-                       const int* y_rows, int glu, hipStream_t st) {
+                       const int* y_rows, int glu, float act_limit, hipStream_t st) {
     constexpr int BM = 128 * WM, BN = 64 * WN;
     // row tiles: a group with rows has 1 + (rows - 1) / tile of them, so groups with rows + M / tile bounds them
     const int m_tiles = offsets ? M / BM + (n_groups < M ? n_groups : M) : (M + BM - 1) / BM;
@@ -192,9 +192,9 @@ static int launch_mfma(const void* X, int ldx, const void* W, long w_group_strid
     SP_REQUIRE((long)m_tiles * n_tiles < (1L << 30), "gemm_mfma: too many tiles");
     dim3 grid((m_tiles * n_tiles + 7) / 8 * 8);
 #define SP_MM(GLUV, TY) do { if (K % MBK == 0) gemm_mfma_kernel<WN, WM, GLUV, true, TY><<<grid, 512, 0, st>>>((const bf16*)X, ldx, \
-        (const bf16*)W, w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, m_tiles, n_tiles, glu); \
+        (const bf16*)W, w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, m_tiles, n_tiles, glu, act_limit); \
     else gemm_mfma_kernel<WN, WM, GLUV, false, TY><<<grid, 512, 0, st>>>((const bf16*)X, ldx, (const bf16*)W, \
-        w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, m_tiles, n_tiles, glu); } while (0)
+        w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, m_tiles, n_tiles, glu, act_limit); } while (0)
     if (glu) { if (y_dtype == SP_BF16) SP_MM(true, bf16); else SP_MM(true, float); }
     else { if (y_dtype == SP_BF16) SP_MM(false, bf16); else SP_MM(false, float); }
 #undef SP_MM
@@ -205,16 +205,17 @@ static int launch_mfma(const void* X, int ldx, const void* W, long w_group_strid
 // `shape`: 0 lets the library choose; 1 = 512 W rows x 128 slots a workgroup, 2 = 256 x 256.
 extern "C" int spite_gemm_mfma(const void* X, int ldx, const void* W, long w_group_stride, void* Y, int y_dtype,
                                int ldy, int M, int N, int K, const int* offsets, int n_groups, const int* a_rows,
-                               const float* a_scale, const int* y_rows, int glu, int shape, hipStream_t st) {
+                               const float* a_scale, const int* y_rows, int glu, float act_limit, int shape, hipStream_t st) {
     SP_REQUIRE(M >= 0 && N > 0 && K > 0 && ldx >= K && ldy >= N, "gemm_mfma: bad sizes M=%d N=%d K=%d", M, N, K);
     SP_REQUIRE(K % 8 == 0 && ldx % 8 == 0, "gemm_mfma: K=%d and the row stride %d must be multiples of 8", K, ldx);
     SP_REQUIRE(((uintptr_t)X & 15) == 0 && ((uintptr_t)W & 15) == 0, "gemm_mfma: operands must be 16-byte aligned");
     SP_REQUIRE(y_dtype == SP_BF16 || y_dtype == SP_F32, "gemm_mfma: output dtype %d", y_dtype);
     SP_REQUIRE(!offsets || n_groups > 0, "gemm_mfma: grouped call without groups");
+    SP_REQUIRE(glu >= 0 && glu <= SP_ACT_LAST && (glu != SP_ACT_CLAMPED || act_limit > 0.f), "gemm_mfma: activation code %d with bound %g", glu, act_limit);
     SP_REQUIRE(shape >= 0 && shape <= 2, "gemm_mfma: tile shape %d", shape);
     if (M == 0) return 0;
     if (shape == 0) shape = (offsets || M <= 128) ? 1 : 2;
     if (shape == 1)
-        return launch_mfma<8, 1>(X, ldx, W, w_group_stride, Y, y_dtype, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu, st);
-    return launch_mfma<4, 2>(X, ldx, W, w_group_stride, Y, y_dtype, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu, st);
+        return launch_mfma<8, 1>(X, ldx, W, w_group_stride, Y, y_dtype, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu, act_limit, st);
+    return launch_mfma<4, 2>(X, ldx, W, w_group_stride, Y, y_dtype, ldy, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu, act_limit, st);
 }

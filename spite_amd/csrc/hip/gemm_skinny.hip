@@ -32,7 +32,7 @@ __global__ __launch_bounds__(NW * 64)
 void gemm_skinny_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restrict__ W, long w_group_stride,
                         TY* __restrict__ Y, int ldy, int M, int N, int K,
                         const int* __restrict__ offsets, int n_groups, const int* __restrict__ a_rows,
-                        const float* __restrict__ a_scale, const int* __restrict__ y_rows, int act) {
+                        const float* __restrict__ a_scale, const int* __restrict__ y_rows, int act, float act_limit) {
     constexpr int RA = GLU ? 2 * R : R;        // A tiles per wave
     constexpr int KB = 32 * S;                 // k elements per block
     constexpr int J = RA * G * 4;              // partial sums per lane
@@ -156,7 +156,7 @@ void gemm_skinny_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restr
             if (GLU) u += red[(w * J + j + JO) * 64 + l];
         }
         if (a_scale) { const float sc = a_scale[s]; v *= sc; u *= sc; }
-        if (GLU) v = sp_gate_act(v, act, true) * u;
+        if (GLU) v = sp_gated(v, u, act, act_limit, true);
         else if (act < 0) v = sp_unary(v, -act, true);                 // a plain product with an activation of its own
         const size_t yr = y_rows ? (size_t)y_rows[s] : (size_t)s;
         Y[yr * ldy + n] = from_f32<TY>(v);
@@ -166,6 +166,7 @@ void gemm_skinny_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restr
 // The activation of the product that the calling thread is launching: the gate's code, or minus the
 // code of a plain product's own activation (set by the entry point).
 static thread_local int g_skinny_act = 0;
+static thread_local float g_skinny_limit = 0.f;      // the activation's bound, where it has one
 
 template <int R, int G, int S, int NW>
 static int launch_skinny(const void* X, int ldx, const void* W, long wgs, void* Y, int y_dtype, int ldy, int M, int N,
@@ -186,7 +187,7 @@ static int launch_skinny(const void* X, int ldx, const void* W, long wgs, void* 
         if (sh > 48 * 1024) { hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)sh); \
             if (e != hipSuccess) return sp_fail("gemm_skinny: cannot get %zu bytes of LDS: %s", sh, hipGetErrorString(e)); } \
         kern<<<grid, NW * 64, sh, st>>>((const bf16*)X, ldx, (const bf16*)W, wgs, (TY*)Y, ldy, M, N, K, offsets, \
-                                        n_groups, a_rows, a_scale, y_rows, g_skinny_act); } while (0)
+                                        n_groups, a_rows, a_scale, y_rows, g_skinny_act, g_skinny_limit); } while (0)
     if (glu) { if (y_dtype == SP_BF16) SP_SK(true, bf16); else SP_SK(true, float); }
     else { if (y_dtype == SP_BF16) SP_SK(false, bf16); else SP_SK(false, float); }
 #undef SP_SK
@@ -199,13 +200,15 @@ static int launch_skinny(const void* X, int ldx, const void* W, long wgs, void* 
 // this hold rows (0: no promise); the grid is cut to the row tiles that can exist.
 extern "C" int spite_gemm_skinny(const void* X, int ldx, const void* W, long w_group_stride, void* Y, int y_dtype,
                                  int ldy, int M, int N, int K, const int* offsets, int n_groups, const int* a_rows,
-                                 const float* a_scale, const int* y_rows, int glu, int max_rows, int variant,
+                                 const float* a_scale, const int* y_rows, int glu, float act_limit, int max_rows, int variant,
                                  int w_tiled, int live_groups, hipStream_t st) {
     SP_REQUIRE(M >= 0 && N > 0 && K > 0 && ldx >= K && ldy >= N, "gemm_skinny: bad sizes M=%d N=%d K=%d", M, N, K);
     const int unary = glu >> 4;
     glu &= 15;
     SP_REQUIRE(!(glu && unary) && unary <= SP_UNARY_TANH, "gemm_skinny: activation code %d", glu | (unary << 4));
+    SP_REQUIRE(glu <= SP_ACT_LAST && (glu != SP_ACT_CLAMPED || act_limit > 0.f), "gemm_skinny: activation code %d with bound %g", glu, act_limit);
     g_skinny_act = glu ? glu : -unary;
+    g_skinny_limit = act_limit;
     SP_REQUIRE(K % 8 == 0 && ldx % 8 == 0, "gemm_skinny: K=%d and the row stride %d must be multiples of 8", K, ldx);
     SP_REQUIRE(((uintptr_t)X & 15) == 0 && ((uintptr_t)W & 15) == 0, "gemm_skinny: operands must be 16-byte aligned");
     SP_REQUIRE(y_dtype == SP_BF16 || y_dtype == SP_F32, "gemm_skinny: output dtype %d", y_dtype);

@@ -39,7 +39,7 @@ void gemm_tiled_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restri
                        TY* __restrict__ Y, int ldy, int M, int N, int K,
                        const int* __restrict__ offsets, int n_groups, const int* __restrict__ a_rows,
                        const float* __restrict__ a_scale, const int* __restrict__ y_rows, int m_tiles, int n_tiles,
-                       int k_splits, size_t split_stride, int act) {
+                       int k_splits, size_t split_stride, int act, float act_limit) {
     static_assert(WN * WM == 8, "eight waves");
     constexpr int WS = 16 * NB;                     // slots of a wave: NB slot tiles
     constexpr int BM = WS * WM, BN = 64 * WN;
@@ -267,7 +267,7 @@ void gemm_tiled_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restri
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const float gv = acc[a][b][i] * sc, uv = acc[a + TG][b][i] * sc;
-                    v[i] = sp_gate_act(gv, act, true) * uv;
+                    v[i] = sp_gated(gv, uv, act, act_limit, true);
                 }
                 put4(yrow, ncol[a] + q * 4, v);
             }
@@ -290,6 +290,7 @@ void gemm_tiled_kernel(const bf16* __restrict__ X, int ldx, const bf16* __restri
 // The gate's activation of the gated product that the calling thread is launching (set by the
 // entry point; the launchers below hand it to the kernel).
 static thread_local int g_gate_act = SP_ACT_SILU;
+static thread_local float g_gate_limit = 0.f;          // the activation's bound, where it has one
 
 template <int WN, int WM, int NB, bool GLU, typename TY, bool NTW = false>
 static int launch_tiled_kernel(const void* X, int ldx, const void* W, long w_group_stride, void* Y, int ldy, int M, int N,
@@ -316,11 +317,11 @@ static int launch_tiled_kernel(const void* X, int ldx, const void* W, long w_gro
     if (offsets)
         gemm_tiled_kernel<WN, WM, NB, GLU, TY, NTW, true><<<grid, 512, sh, st>>>(
             (const bf16*)X, ldx, (const bf16*)W, w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale,
-            y_rows, m_tiles, n_tiles, k_splits, split_stride, g_gate_act);
+            y_rows, m_tiles, n_tiles, k_splits, split_stride, g_gate_act, g_gate_limit);
     else
         gemm_tiled_kernel<WN, WM, NB, GLU, TY, NTW, false><<<grid, 512, sh, st>>>(
             (const bf16*)X, ldx, (const bf16*)W, w_group_stride, (TY*)Y, ldy, M, N, K, offsets, n_groups, a_rows, a_scale,
-            y_rows, m_tiles, n_tiles, k_splits, split_stride, g_gate_act);
+            y_rows, m_tiles, n_tiles, k_splits, split_stride, g_gate_act, g_gate_limit);
     SP_LAUNCH_CHECK("gemm_tiled");
     return 0;
 }
@@ -390,7 +391,7 @@ extern "C" int spite_gemm_tiled_split(const void* X, int ldx, const void* W, voi
 // products only).
 extern "C" int spite_gemm_tiled(const void* X, int ldx, const void* W, long w_group_stride, void* Y, int y_dtype,
                                 int ldy, int M, int N, int K, const int* offsets, int n_groups, const int* a_rows,
-                                const float* a_scale, const int* y_rows, int glu, int shape, hipStream_t st) {
+                                const float* a_scale, const int* y_rows, int glu, float act_limit, int shape, hipStream_t st) {
     SP_REQUIRE(M >= 0 && N > 0 && K > 0 && ldx >= K && ldy >= N, "gemm_tiled: bad sizes M=%d N=%d K=%d", M, N, K);
     SP_REQUIRE(K % 64 == 0 && N % 16 == 0, "gemm_tiled: operand order needs K=%d a multiple of 64 and N=%d of 16", K, N);
     SP_REQUIRE(ldx % 8 == 0, "gemm_tiled: the row stride %d must be a multiple of 8", ldx);
@@ -401,7 +402,9 @@ extern "C" int spite_gemm_tiled(const void* X, int ldx, const void* W, long w_gr
     const int unary = glu >> 4;
     glu &= 15;
     SP_REQUIRE(!(glu && unary) && unary <= SP_UNARY_TANH, "gemm_tiled: activation code %d", glu | (unary << 4));
+    SP_REQUIRE(glu <= SP_ACT_LAST && (glu != SP_ACT_CLAMPED || act_limit > 0.f), "gemm_tiled: activation code %d with bound %g", glu, act_limit);
     g_gate_act = glu ? glu : (unary ? -unary : SP_ACT_SILU);
+    g_gate_limit = act_limit;
     if (M == 0) return 0;
     if (shape == 0) {
         // Tiles come in whole numbers per CU: a plain product whose 128-row tiles leave many of the

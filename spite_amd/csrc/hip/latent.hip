@@ -22,6 +22,9 @@
 //       turn, adjacent pairs (2i, 2i+1) by pos * inv_freq[i]; the rest pass);
 //   (own) the cache row slot_map[t]: the latent, RMS-normed with weight `w_norm`, then the
 //       rotated shared key part;
+//   (with `cq_out`) cq_out[t] = the query latent, `Q` elements of the row `cq_raw`, RMS-normed with weight `w_cq`:
+//       queries that go through a latent of their own are projected from it after this kernel (`qd` is then
+//       null, or comes in a second call for its rotated parts);
 //   rows_th[h*T + t] = t*H + h and offsets_h[h] = h*T: the row list by which a grouped product
 //       with one group per head walks rows that lie token by token.
 // Angles, rotation and norm are fp32; sine and cosine are the accurate routines.
@@ -31,7 +34,8 @@ void latent_prepare_kernel(const T* __restrict__ qd, int ldq, const T* __restric
                            const int* __restrict__ positions, const int* __restrict__ slot_map,
                            const float* __restrict__ inv_freq, const float* __restrict__ w_norm, float eps,
                            int H, int n, int r, int R, int rot_dims, int own,
-                           int* __restrict__ rows_th, int* __restrict__ offsets_h, int T_all) {
+                           int* __restrict__ rows_th, int* __restrict__ offsets_h, int T_all,
+                           const T* __restrict__ cq_raw, int ld_cq, const float* __restrict__ w_cq, T* __restrict__ cq_out, int Q) {
     __shared__ float red[4];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int Dk = R + r, hw = n + r;
@@ -45,9 +49,16 @@ void latent_prepare_kernel(const T* __restrict__ qd, int ldq, const T* __restric
         const float u = to_f32<T>(part[2 * i]), v = to_f32<T>(part[2 * i + 1]);
         return (e & 1) ? v * cs + u * sn : u * cs - v * sn;
     };
-    for (int i = tid; i < H * r; i += 256) {
+    if (qd) for (int i = tid; i < H * r; i += 256) {
         const int h = i / r, e = i - h * r;
         qa[((size_t)t * H + h) * Dk + R + e] = from_f32<T>(turned(row + (size_t)h * hw + n, e));
+    }
+    if (cq_out) {
+        const T* cq = cq_raw + (size_t)t * ld_cq;
+        float sq = 0.f;
+        for (int e = tid; e < Q; e += 256) { const float x = to_f32<T>(cq[e]); sq += x * x; }
+        const float scale = 1.0f / sqrtf(block_sum<256>(sq, red) / (float)Q + eps);
+        for (int e = tid; e < Q; e += 256) cq_out[(size_t)t * Q + e] = from_f32<T>(to_f32<T>(cq[e]) * scale * w_cq[e]);
     }
     if (own) {
         const T* dkv = dkv_all + (size_t)t * ld_dkv;
@@ -68,19 +79,23 @@ void latent_prepare_kernel(const T* __restrict__ qd, int ldq, const T* __restric
 extern "C" int spite_latent_prepare(const void* qd, int ldq, const void* dkv, int ld_dkv, void* qa, void* kv_pages, int dtype, const int* positions,
                                     const int* slot_map, const float* inv_freq, const float* w_norm, float eps,
                                     int T, int H, int n, int r, int R, int rot_dims, int own,
-                                    int* rows_th, int* offsets_h, hipStream_t st) {
+                                    int* rows_th, int* offsets_h, const void* cq_raw, int ld_cq, const float* w_cq, void* cq_out,
+                                    int Q, hipStream_t st) {
     SP_REQUIRE(T >= 0 && H > 0 && n > 0 && r >= 0 && R > 0, "latent_prepare: bad sizes T=%d H=%d n=%d r=%d R=%d", T, H, n, r, R);
     SP_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= r, "latent_prepare: %d turning elements of %d", rot_dims, r);
-    SP_REQUIRE(ldq >= H * (n + r) && (!own || ld_dkv >= R + r), "latent_prepare: rows of %d or %d are too short", ldq, ld_dkv);
+    SP_REQUIRE(!cq_out || (cq_raw && w_cq && Q > 0 && ld_cq >= Q && eps > 0.f), "latent_prepare: query latent of %d in rows of %d", Q, ld_cq);
+    SP_REQUIRE(rot_dims == 0 || inv_freq, "latent_prepare: rotation needs a frequency table");
+    SP_REQUIRE(!qd || qa, "latent_prepare: queries without an output");
+    SP_REQUIRE((!qd || ldq >= H * (n + r)) && (!own || ld_dkv >= R + r), "latent_prepare: rows of %d or %d are too short", ldq, ld_dkv);
     SP_REQUIRE(!own || (dkv && kv_pages && slot_map && w_norm && eps > 0.f), "latent_prepare: the cache row needs pages, slots and the norm");
     SP_REQUIRE((long)T * H < (1L << 31), "latent_prepare: too many rows");
     if (T == 0) return 0;
     if (dtype == SP_F32)
         latent_prepare_kernel<float><<<T, 256, 0, st>>>((const float*)qd, ldq, (const float*)dkv, ld_dkv, (float*)qa, (float*)kv_pages, positions, slot_map,
-            inv_freq, w_norm, eps, H, n, r, R, rot_dims, own, rows_th, offsets_h, T);
+            inv_freq, w_norm, eps, H, n, r, R, rot_dims, own, rows_th, offsets_h, T, (const float*)cq_raw, ld_cq, w_cq, (float*)cq_out, Q);
     else if (dtype == SP_BF16)
         latent_prepare_kernel<bf16><<<T, 256, 0, st>>>((const bf16*)qd, ldq, (const bf16*)dkv, ld_dkv, (bf16*)qa, (bf16*)kv_pages, positions, slot_map,
-            inv_freq, w_norm, eps, H, n, r, R, rot_dims, own, rows_th, offsets_h, T);
+            inv_freq, w_norm, eps, H, n, r, R, rot_dims, own, rows_th, offsets_h, T, (const bf16*)cq_raw, ld_cq, w_cq, (bf16*)cq_out, Q);
     else return sp_fail("latent_prepare: unknown dtype %d", dtype);
     SP_LAUNCH_CHECK("latent_prepare");
     return 0;

@@ -18,7 +18,7 @@ from . import build
 F32, BF16 = 0, 1
 VIS = build.visibility_codes()      # "full", "chunk", "window": name -> code
 # the gate's activation of a gated product act(gate) * up, as the kernels number them (True: silu)
-GATE_ACTS = {False: 0, None: 0, True: 1, "silu": 1, "gelu_tanh": 2, "relu": 3}
+GATE_ACTS = {False: 0, None: 0, True: 1, "silu": 1, "gelu_tanh": 2, "relu": 3, "clamped": 4}
 # an activation of a plain product's own (no gate), as the kernels number them; the bf16 weight-stream and
 # tiled products take it in their epilogue, in the bits above the gate's code
 UNARY_ACTS = {"gelu": 1, "gelu_tanh": 2, "silu": 3, "tanh": 4}
@@ -26,6 +26,17 @@ UNARY_ACTS = {"gelu": 1, "gelu_tanh": 2, "silu": 3, "tanh": 4}
 
 class KernelError(RuntimeError):
     pass
+
+
+def gate_code(glu):
+    """(code, bound) of a gated product's activation: a name of ``GATE_ACTS`` or, for the one that has a bound,
+    ``("clamped", limit)``: min(gate, limit) * sigmoid(1.702 min(gate, limit)) * (clamp(up, -limit, limit) + 1)."""
+    name, limit = glu if isinstance(glu, tuple) else (glu, 0.0)
+    if name not in GATE_ACTS:
+        raise KernelError(f"gated product: activation {name!r} (known: {sorted(k for k in GATE_ACTS if isinstance(k, str))})")
+    if (name == "clamped") != (limit > 0.0):
+        raise KernelError(f"gated product: activation {name!r} with bound {limit} (clamped alone has one, above 0)")
+    return GATE_ACTS[name], float(limit)
 
 
 _lib = None
@@ -46,28 +57,28 @@ def lib():
             "spite_convert": [P, I, P, I, c_size_t, P],
             "spite_add_into": [P, P, c_size_t, P],
             "spite_randn_fill": [P, I, c_size_t, ctypes.c_ulonglong, ctypes.c_ulonglong, F, F, P],
-            "spite_gemm_generic": [P, I, P, L, I, P, I, I, I, I, I, P, I, P, P, P, I, P],
+            "spite_gemm_generic": [P, I, P, L, I, P, I, I, I, I, I, P, I, P, P, P, I, F, P],
             "spite_attn_generic": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, F, F, P, I, P],
             "spite_sample_rows": [P, I, I, I, P, P, P, P],
             "spite_filter_rows": [P, I, I, I, P, P, P, P],
-            "spite_gemm_skinny": [P, I, P, L, P, I, I, I, I, I, P, I, P, P, P, I, I, I, I, I, P],
-            "spite_attn_decode": [P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, I, I, P, P],
-            "spite_gemm_mfma": [P, I, P, L, P, I, I, I, I, I, P, I, P, P, P, I, I, P],
-            "spite_gemm_tiled": [P, I, P, L, P, I, I, I, I, I, P, I, P, P, P, I, I, P],
+            "spite_gemm_skinny": [P, I, P, L, P, I, I, I, I, I, P, I, P, P, P, I, F, I, I, I, I, P],
+            "spite_attn_decode": [P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, I, I, P, I, I, P, I, P],
+            "spite_gemm_mfma": [P, I, P, L, P, I, I, I, I, I, P, I, P, P, P, I, F, I, P],
+            "spite_gemm_tiled": [P, I, P, L, P, I, I, I, I, I, P, I, P, P, P, I, F, I, P],
             "spite_gemm_tiled_split": [P, I, P, P, I, I, I, I, I, I, P, P],
-            "spite_attn_prefill": [P, P, P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, F, F, P, I, I, P, P],
+            "spite_attn_prefill": [P, P, P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, F, F, P, I, I, P, I, I, P, I, P],
             "spite_attn_prefill_splits": [P, I, I, I, L],
             "spite_argmax_rows": [P, I, I, I, P, P, P, P],
             "spite_stream_read": [P, c_size_t, P, I, P],
             "spite_mfma_loop": [P, I, I, F, P],
-            "spite_latent_prepare": [P, I, P, I, P, P, I, P, P, P, P, F, I, I, I, I, I, I, I, P, P, P],
+            "spite_latent_prepare": [P, I, P, I, P, P, I, P, P, P, P, F, I, I, I, I, I, I, I, P, P, P, I, P, P, I, P],
             "spite_attn_latent_generic": [P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, F, P],
             "spite_attn_latent_mfma": [P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, F, P, I, I, P],
-            "spite_router_topk": [P, P, P, P, I, I, I, I, I, P],
-            "spite_moe_combine": [P, P, P, P, I, I, I, P],
+            "spite_router_topk": [P, P, P, P, I, I, I, I, I, I, I, I, P],
+            "spite_moe_combine": [P, P, P, P, I, P, I, I, I, P],
             "spite_gated_rows": [P, I, P, P, I, I, I, P, I, I, P],
-            "spite_qkv_prepare": [P, I, I, P, P, P, F, P, P, P, P, P, P, I, F, P, I, I, I, I, I, I, I, I, I, I, I, F, I, I, P],
-            "spite_attn_wide": [P, P, P, P, I, I, P, P, P, I, I, I, I, I, I, I, I, I, I, F, I, I, P, P, P],
+            "spite_qkv_prepare": [P, I, I, P, P, P, F, P, P, P, P, P, P, I, F, P, I, I, I, I, I, I, I, I, I, I, I, F, I, I, P, I, F, P],
+            "spite_attn_wide": [P, P, P, P, I, I, P, P, P, I, I, I, I, I, I, I, I, I, I, F, I, I, P, P, I, P, I, P],
             "spite_attn_finish": [P, I, P, I, P, P, P, I, I, I, I, I, F, F, F, P],
             "spite_token_shift": [P, P, I, P, P, P, P, P, I, I, I, P],
             "spite_act_rows": [P, I, c_size_t, I, P],
@@ -129,9 +140,9 @@ def _ptr_rows(t, name):
     return _ptr(t, name)
 
 
-def _check_pages(k_pages, v_pages, G, page_size, hd, what, value_heads=None):
-    """Key pages [n, G, page_size, hd]; value pages transposed, [n, G (or value_heads), hd, page_size]."""
-    if (tuple(k_pages.shape[1:]) != (G, page_size, hd) or tuple(v_pages.shape[1:]) != (value_heads or G, hd, page_size)
+def _check_pages(k_pages, v_pages, G, page_size, hd, what, value_heads=None, v_dim=None):
+    """Key pages [n, G, page_size, hd]; value pages transposed, [n, G (or value_heads), hd (or v_dim), page_size]."""
+    if (tuple(k_pages.shape[1:]) != (G, page_size, hd) or tuple(v_pages.shape[1:]) != (value_heads or G, v_dim or hd, page_size)
             or k_pages.shape[0] != v_pages.shape[0]):
         raise KernelError(f"{what}: key pages {tuple(k_pages.shape)}, value pages {tuple(v_pages.shape)} for "
                           f"G={G} page={page_size} hd={hd}")
@@ -306,9 +317,9 @@ def randn_fill(t, seed: int, key: int, mean: float = 0.0, std: float = 1.0):
 
 
 def gemm_generic(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_scale=None, y_rows=None,
-                 glu=False):
+                 glu=False, act_limit=0.0):
     """Y = A . W^T (see gemm_generic.hip).  a [rows,K]; w [groups, N or 2N, K] or [N or 2N, K];
-    y [rows,N]."""
+    y [rows,N].  ``glu``: the gate's activation as ``gate_code`` numbers it, ``act_limit`` its bound."""
     if a.shape[-1] != K or y.shape[-1] != N:
         raise KernelError(f"gemm: a {tuple(a.shape)}, y {tuple(y.shape)} for N={N} K={K}")
     rows_w = 2 * N if glu else N
@@ -331,7 +342,7 @@ def gemm_generic(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_s
         _ptr_rows(a, "a"), a.stride(0) if a.dim() == 2 else K, _ptr(w, "w"), rows_w * K, dtype_code(a.dtype),
         _ptr_rows(y, "y"), dtype_code(y.dtype), y.stride(0), M, N, K, _ptr(offsets, "offsets", torch.int32, True), n_groups,
         _ptr(a_rows, "a_rows", torch.int32, True), _ptr(a_scale, "a_scale", torch.float32, True),
-        _ptr(y_rows, "y_rows", torch.int32, True), int(glu), _stream()), "gemm")
+        _ptr(y_rows, "y_rows", torch.int32, True), int(glu), float(act_limit), _stream()), "gemm")
 
 
 def attn_generic(q, k_pages, v_pages, out, positions, seq_of_token, block_table, T, H, G, hd, page_size,
@@ -404,7 +415,7 @@ def _gemm_checks(a, w, y, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, g
 
 
 def gemm_skinny(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_scale=None, y_rows=None,
-                glu=False, max_rows=None, variant=0, tiled=False, live_groups=0, act=None):
+                glu=False, max_rows=None, variant=0, tiled=False, live_groups=0, act=None, act_limit=0.0):
     """Weight-streaming bf16 product for few rows (see gemm_skinny.hip); arguments as gemm_generic.
     ``max_rows``: the most rows a group can bring (default M).  ``tiled``: w is in MFMA operand
     order (``operand_order``).  ``live_groups``: a promise that at most this many groups hold rows
@@ -415,7 +426,7 @@ def gemm_skinny(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_sc
     _check(lib().spite_gemm_skinny(
         _ptr_rows(a, "a"), a.stride(0), _ptr(w, "w"), rows_w * K, _ptr_rows(y, "y"), dtype_code(y.dtype), y.stride(0),
         M, N, K, _ptr(offsets, "offsets", torch.int32, True), n_groups, _ptr(a_rows, "a_rows", torch.int32, True),
-        _ptr(a_scale, "a_scale", torch.float32, True), _ptr(y_rows, "y_rows", torch.int32, True), _act_code(glu, act),
+        _ptr(a_scale, "a_scale", torch.float32, True), _ptr(y_rows, "y_rows", torch.int32, True), _act_code(glu, act), float(act_limit),
         int(max_rows if max_rows is not None else M), int(variant), int(bool(tiled)), int(live_groups), _stream()),
         "gemm_skinny")
 
@@ -453,26 +464,41 @@ def kv_operand_order(k_pages, v_pages):
     return k.contiguous().view(n, G, ps, hd), v.contiguous().view(n, Gv, hd, ps)
 
 
+#: (key width, value width) that the MFMA kernels ``attn_decode`` and ``attn_prefill`` take
+ATTN_WIDTHS = ((64, 32), (64, 64), (128, 64), (128, 128))
+
+
+def attn_stored_width(D, Vd):
+    """The width that keys of D are stored with (zeros behind their own elements) so that the MFMA attention
+    kernels take them beside values of Vd, or None where they take no such pair."""
+    fits = [k for k, v in ATTN_WIDTHS if v == Vd and k >= D]
+    return min(fits) if fits else None
+
+
 def attn_decode_workspace(T, H, hd, n_splits) -> int:
-    """Bytes of scratch that attn_decode needs."""
+    """Bytes of scratch that attn_decode needs (``hd``: the values' width)."""
     return T * H * n_splits * (hd + 2) * 4
 
 
 def attn_decode(q, k_pages, v_pages, out, workspace, positions, seq_of_token, block_table, T, H, G, hd,
-                page_size, vis, span, scale, n_splits, softcap=0.0, slopes=None, value_heads=None, sinks=None):
+                page_size, vis, span, scale, n_splits, softcap=0.0, slopes=None, value_heads=None, sinks=None, v_dim=None,
+                keep=0, dist_bias=None):
     """Split-KV decode attention on MFMA (bf16; head sizes 64 and 128; pages of a multiple of 32
     keys, in operand order): every row of q is one query against its request's cache.
     ``value_heads``: the value pages hold fewer heads than the key pages (kv head g reads value
     head g % value_heads).  ``sinks`` (fp32 [H] or None): one more term exp(sinks[h]) in every
-    softmax's denominator."""
+    softmax's denominator.  Here and in ``attn_prefill``: ``v_dim``: the values' width where it is not ``hd``
+    (``ATTN_WIDTHS``); ``keep``: with a chunk or a window the request's first so many keys are read too;
+    ``dist_bias`` (fp32 [H, n] or None): dist_bias[h, min(p - j, n - 1)] is added to the scaled score."""
+    Vd = int(v_dim or hd)
     if q.dtype != torch.bfloat16:
         raise KernelError(f"attn_decode: bfloat16 only, got {q.dtype}")
-    if q.numel() < T * H * hd or out.numel() < T * H * hd:
+    if q.numel() < T * H * hd or out.numel() < T * H * Vd:
         raise KernelError("attn_decode: q or out too small")
-    _check_pages(k_pages, v_pages, G, page_size, hd, "attn_decode", value_heads)
+    _check_pages(k_pages, v_pages, G, page_size, hd, "attn_decode", value_heads, Vd)
     if block_table.dim() != 2 or positions.numel() < T or seq_of_token.numel() < T:
         raise KernelError("attn_decode: metadata too small")
-    if workspace.numel() * workspace.element_size() < attn_decode_workspace(T, H, hd, n_splits):
+    if workspace.numel() * workspace.element_size() < attn_decode_workspace(T, H, Vd, n_splits):
         raise KernelError("attn_decode: workspace too small")
     dt = torch.bfloat16
     _check(lib().spite_attn_decode(
@@ -480,11 +506,12 @@ def attn_decode(q, k_pages, v_pages, out, workspace, positions, seq_of_token, bl
         _ptr(workspace, "workspace"), _ptr(positions, "positions", torch.int32),
         _ptr(seq_of_token, "seq_of_token", torch.int32), _ptr(block_table, "block_table", torch.int32),
         block_table.shape[1], T, H, G, hd, page_size, VIS[vis], int(span or 0), float(scale), float(softcap),
-        _slopes(slopes, H), int(n_splits), int(value_heads or 0), _slopes(sinks, H), _stream()), "attn_decode")
+        _slopes(slopes, H), int(n_splits), int(value_heads or 0), _slopes(sinks, H), Vd, int(keep), *_dist_bias(dist_bias, H),
+        _stream()), "attn_decode")
 
 
 def gemm_mfma(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_scale=None, y_rows=None, glu=False,
-              shape=0):
+              shape=0, act_limit=0.0):
     """Tiled bf16 MFMA product for many rows (see gemm_mfma.hip); arguments as gemm_generic."""
     rows_w = _gemm_checks(a, w, y, M, N, K, offsets, n_groups, a_rows, a_scale, y_rows, glu, "gemm_mfma")
     if a.dtype != torch.bfloat16 or w.dtype != torch.bfloat16:
@@ -493,7 +520,7 @@ def gemm_mfma(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_scal
         _ptr_rows(a, "a"), a.stride(0), _ptr(w, "w"), rows_w * K, _ptr_rows(y, "y"), dtype_code(y.dtype), y.stride(0),
         M, N, K, _ptr(offsets, "offsets", torch.int32, True), n_groups, _ptr(a_rows, "a_rows", torch.int32, True),
         _ptr(a_scale, "a_scale", torch.float32, True), _ptr(y_rows, "y_rows", torch.int32, True), int(glu),
-        int(shape), _stream()), "gemm_mfma")
+        float(act_limit), int(shape), _stream()), "gemm_mfma")
 
 
 def operand_order(w: torch.Tensor) -> torch.Tensor:
@@ -533,7 +560,7 @@ def cu_count() -> int:
 
 
 def gemm_tiled(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_scale=None, y_rows=None, glu=False,
-               shape=0, part=None, act=None):
+               shape=0, part=None, act=None, act_limit=0.0):
     """Tiled bf16 MFMA product for many rows over weights in operand order (``operand_order``;
     see gemm_tiled.hip); arguments as gemm_generic.  ``part`` (fp32 ``[runs, M, N]``, plain
     products only): the sum over k is cut into ``runs`` runs, each a workgroup of its own, whose
@@ -556,7 +583,7 @@ def gemm_tiled(a, w, y, M, N, K, *, offsets=None, n_groups=1, a_rows=None, a_sca
         _ptr_rows(a, "a"), a.stride(0), _ptr(w, "w"), rows_w * K, _ptr_rows(y, "y"), dtype_code(y.dtype), y.stride(0),
         M, N, K, _ptr(offsets, "offsets", torch.int32, True), n_groups, _ptr(a_rows, "a_rows", torch.int32, True),
         _ptr(a_scale, "a_scale", torch.float32, True), _ptr(y_rows, "y_rows", torch.int32, True), _act_code(glu, act),
-        int(shape), _stream()), "gemm_tiled")
+        float(act_limit), int(shape), _stream()), "gemm_tiled")
 
 
 def attn_prefill_splits(counts, H, G, max_keys) -> int:
@@ -567,14 +594,14 @@ def attn_prefill_splits(counts, H, G, max_keys) -> int:
 
 
 def attn_prefill_workspace(counts, H, G, hd, n_splits) -> int:
-    """Bytes of fp32 scratch that ``attn_prefill`` needs for ``n_splits`` > 1 (none for 1)."""
+    """Bytes of fp32 scratch that ``attn_prefill`` needs for ``n_splits`` > 1 (none for 1); ``hd``: the values' width."""
     counts = np.ascontiguousarray(counts, dtype=np.int32)
     return int(lib().spite_attn_prefill_workspace(counts.ctypes.data, int(counts.size), H, G, hd, int(n_splits)))
 
 
 def attn_prefill(q, k_pages, v_pages, out, positions, cu_seqlens, counts, block_table,
                  H, G, hd, page_size, vis, span, scale, n_splits=1, scratch=None, softcap=0.0, slopes=None, value_heads=None,
-                 sinks=None):
+                 sinks=None, v_dim=None, keep=0, dist_bias=None):
     """Prefill attention on MFMA (bf16; head sizes 64 and 128; pages of a multiple of 32 keys, in
     operand order).
     ``counts``: the number of query tokens of every request of the step, on the host, in the
@@ -583,22 +610,23 @@ def attn_prefill(q, k_pages, v_pages, out, positions, cu_seqlens, counts, block_
     ``attn_prefill_workspace`` bytes) then holds their partial results.
     ``slopes`` (fp32 [H] or None): a bias slopes[head] * (key position - query position) on the
     scaled scores, before the cap.  ``sinks`` (fp32 [H] or None): one more term exp(sinks[h]) in
-    every softmax's denominator."""
+    every softmax's denominator.  ``v_dim``, ``keep``, ``dist_bias``: as ``attn_decode``."""
+    Vd = int(v_dim or hd)
     if q.dtype != torch.bfloat16:
         raise KernelError(f"attn_prefill: bfloat16 only, got {q.dtype}")
     counts = np.ascontiguousarray(counts, dtype=np.int32)
     n_seqs = int(counts.size)
     T = int(counts.sum())
-    if q.numel() < T * H * hd or out.numel() < T * H * hd:
+    if q.numel() < T * H * hd or out.numel() < T * H * Vd:
         raise KernelError("attn_prefill: q or out too small")
-    _check_pages(k_pages, v_pages, G, page_size, hd, "attn_prefill", value_heads)
+    _check_pages(k_pages, v_pages, G, page_size, hd, "attn_prefill", value_heads, Vd)
     if block_table.dim() != 2 or block_table.shape[0] < n_seqs or positions.numel() < T:
         raise KernelError("attn_prefill: metadata too small")
     if cu_seqlens.numel() < n_seqs + 1:
         raise KernelError("attn_prefill: cu_seqlens shorter than the requests of the step")
     n_splits = int(n_splits)
-    if n_splits > 1 and (scratch is None or scratch.numel() * 4 < attn_prefill_workspace(counts, H, G, hd, n_splits)):
-        raise KernelError(f"attn_prefill: {n_splits} splits need {attn_prefill_workspace(counts, H, G, hd, n_splits)} bytes of scratch")
+    if n_splits > 1 and (scratch is None or scratch.numel() * 4 < attn_prefill_workspace(counts, H, G, Vd, n_splits)):
+        raise KernelError(f"attn_prefill: {n_splits} splits need {attn_prefill_workspace(counts, H, G, Vd, n_splits)} bytes of scratch")
     dt = torch.bfloat16
     _check(lib().spite_attn_prefill(
         _ptr(q, "q", dt), _ptr(k_pages, "k_pages", dt), _ptr(v_pages, "v_pages", dt), _ptr(out, "out", dt),
@@ -606,7 +634,16 @@ def attn_prefill(q, k_pages, v_pages, out, positions, cu_seqlens, counts, block_
         _ptr(positions, "positions", torch.int32), _ptr(cu_seqlens, "cu_seqlens", torch.int32),
         counts.ctypes.data, n_seqs, _ptr(block_table, "block_table", torch.int32), block_table.shape[1],
         H, G, hd, page_size, VIS[vis], int(span or 0), float(scale), float(softcap), _slopes(slopes, H), n_splits,
-        int(value_heads or 0), _slopes(sinks, H), _stream()), "attn_prefill")
+        int(value_heads or 0), _slopes(sinks, H), Vd, int(keep), *_dist_bias(dist_bias, H), _stream()), "attn_prefill")
+
+
+def _dist_bias(table, H):
+    """(pointer, entries a head) of a table of biases by distance."""
+    if table is None:
+        return None, 0
+    if table.dim() != 2 or table.shape[0] != H or table.shape[1] < 1:
+        raise KernelError(f"bias by distance: a table {tuple(table.shape)} for {H} query heads")
+    return _ptr(table, "dist_bias", torch.float32), table.shape[1]
 
 
 def _slopes(slopes, H):
@@ -649,32 +686,48 @@ def mfma_loop(out, steps, gain):
 
 # -------------------------------------------------------------------------------------------- latent attention
 def latent_prepare(qd, dkv, qa, kv_pages, positions, slot_map, inv_freq, w_norm, eps, H, n, r, R, rot_dims, own,
-                   rows_th, offsets_h):
+                   rows_th, offsets_h, query_latent=None):
     """Between the projections and the per-head products of latent attention (see latent.hip):
     qd [T, H*(n+r)]; dkv [T, R+r] (with ``own``); qa [T*H, R+r] receives the rotated query parts; with ``own`` the
     cache row of every token (kv_pages [pages, 1, page_size, R+r]) receives the normed latent and the
     rotated shared key part; rows_th int32 [H*T] and offsets_h int32 [H+1] receive the row list of
-    the per-head products."""
-    T = qd.shape[0]
+    the per-head products.  ``qd`` None: the queries come later (their latent is normed here first) or have no
+    rotated part; qa is left alone.  ``query_latent`` = (raw [T, >= Q] rows, weight fp32 [Q], out [T, Q]): out = the raw
+    rows RMS-normed (the same eps) times the weight."""
+    if qd is None and (dkv is None or not own):
+        raise KernelError("latent_prepare: neither queries nor cache rows to prepare")
+    T = (dkv if qd is None else qd).shape[0]
     Dk = R + r
-    if qd.dim() != 2 or qd.stride(1) != 1 or qd.shape[1] < H * (n + r):
+    Q, raw, w_q, out_q = 0, None, None, None
+    if query_latent is not None:
+        raw, w_q, out_q = query_latent
+        Q = w_q.numel()
+        if raw.dim() != 2 or raw.stride(1) != 1 or raw.shape[0] < T or raw.shape[1] < Q or tuple(out_q.shape) != (T, Q) \
+                or raw.dtype != out_q.dtype or raw.dtype != (dkv if qd is None else qd).dtype:
+            raise KernelError(f"latent_prepare: query latent {tuple(raw.shape)} to {tuple(out_q.shape)} with a weight of {Q}")
+    if qd is None:
+        pass
+    elif qd.dim() != 2 or qd.stride(1) != 1 or qd.shape[1] < H * (n + r):
         raise KernelError(f"latent_prepare: qd {tuple(qd.shape)} for H={H} n={n} r={r} R={R} own={own}")
-    if own and (dkv is None or dkv.dim() != 2 or dkv.stride(1) != 1 or dkv.shape[1] < R + r or dkv.shape[0] < T or dkv.dtype != qd.dtype):
+    if own and (dkv is None or dkv.dim() != 2 or dkv.stride(1) != 1 or dkv.shape[1] < R + r or dkv.shape[0] < T or (qd is not None and dkv.dtype != qd.dtype)):
         raise KernelError(f"latent_prepare: the down-projection's rows do not fit R={R} r={r}")
-    if qa.numel() < T * H * Dk or positions.numel() < T or rows_th.numel() < H * T or offsets_h.numel() < H + 1:
+    if (qd is not None and qa.numel() < T * H * Dk) or positions.numel() < T or rows_th.numel() < H * T or offsets_h.numel() < H + 1:
         raise KernelError("latent_prepare: outputs or positions too small")
-    if inv_freq.numel() < rot_dims // 2:
+    if rot_dims and inv_freq.numel() < rot_dims // 2:
         raise KernelError("latent_prepare: frequency table shorter than the turning pairs")
-    dt = qd.dtype
+    dt = (dkv if qd is None else qd).dtype
     if own:
         if kv_pages.dim() != 4 or kv_pages.shape[1] != 1 or kv_pages.shape[3] != Dk or slot_map.numel() < T or w_norm.numel() != R:
             raise KernelError(f"latent_prepare: pages {tuple(kv_pages.shape)} for rows of {Dk}, or slots / norm weight too small")
     _check(lib().spite_latent_prepare(
-        _ptr_rows(qd, "qd"), qd.stride(0), _ptr_rows(dkv, "dkv") if own else None, dkv.stride(0) if own else 0, _ptr(qa, "qa", dt), _ptr(kv_pages, "kv_pages", dt, not own), dtype_code(dt),
+        _ptr_rows(qd, "qd") if qd is not None else None, qd.stride(0) if qd is not None else 0,
+        _ptr_rows(dkv, "dkv") if own else None, dkv.stride(0) if own else 0, _ptr(qa, "qa", dt, qd is None), _ptr(kv_pages, "kv_pages", dt, not own), dtype_code(dt),
         _ptr(positions, "positions", torch.int32), _ptr(slot_map, "slot_map", torch.int32, not own),
-        _ptr(inv_freq, "inv_freq", torch.float32), _ptr(w_norm, "w_norm", torch.float32, not own), float(eps),
+        _ptr(inv_freq, "inv_freq", torch.float32, rot_dims == 0), _ptr(w_norm, "w_norm", torch.float32, not own), float(eps),
         T, H, n, r, R, int(rot_dims), int(bool(own)), _ptr(rows_th, "rows_th", torch.int32),
-        _ptr(offsets_h, "offsets_h", torch.int32), _stream()), "latent_prepare")
+        _ptr(offsets_h, "offsets_h", torch.int32),
+        _ptr_rows(raw, "query latent") if Q else None, raw.stride(0) if Q else 0, _ptr(w_q, "query latent's weight", torch.float32, not Q),
+        _ptr(out_q, "query latent's output", dt, not Q), Q, _stream()), "latent_prepare")
 
 
 def _latent_checks(q, kv_pages, out, positions, seq_of_token, block_table, T, H, Dk, R, what):
@@ -699,34 +752,44 @@ def attn_latent_generic(q, kv_pages, out, positions, seq_of_token, block_table, 
 
 
 # -------------------------------------------------------------------------------------------- several experts a token
-ROUTER_SCORING = {"sigmoid": 0, "softmax_taken": 1}
+ROUTER_SCORING = {"sigmoid": 0, "softmax_taken": 1, "softmax": 2}
 
 
-def router_topk(logits, bias, expert, weight, top, renorm=False, scoring="sigmoid"):
+def router_topk(logits, bias, expert, weight, top, renorm=False, scoring="sigmoid", groups=None, n_experts=None):
     """From fp32 router logits [T, E]: scores sigmoid(z); the ``top`` experts with the largest
     score + bias (bias fp32 [E] or None; lowest index among equals) into expert[T*top], their
     scores (without the bias; divided by their sum with ``renorm``) into weight[T*top].  With
     ``scoring`` = ``softmax_taken`` the choice goes by z + bias and the weights are the softmax over the
-    taken experts' logits."""
-    T, E = logits.shape
+    taken experts' logits; ``softmax``: scores softmax(z) over all experts, the rest as with sigmoid.  ``groups`` =
+    (count, keep): only experts of the ``keep`` groups (``count`` equal groups of neighbours) whose largest choice
+    value is largest can be taken.  ``n_experts``: the logits are the first so many columns of the rows."""
+    T, E = logits.shape[0], int(n_experts or logits.shape[1])
+    count, keep = (1, 1) if groups is None else (int(groups[0]), int(groups[1]))
+    if E > logits.shape[1]:
+        raise KernelError(f"router_topk: {E} experts in rows of {logits.shape[1]}")
     if scoring not in ROUTER_SCORING:
         raise KernelError(f"router_topk: scoring {scoring!r} (known: {sorted(ROUTER_SCORING)})")
     if expert.numel() < T * top or weight.numel() < T * top or (bias is not None and bias.numel() != E):
         raise KernelError("router_topk: outputs too small or bias of the wrong size")
     _check(lib().spite_router_topk(_ptr(logits, "logits", torch.float32), _ptr(bias, "bias", torch.float32, True),
                                    _ptr(expert, "expert", torch.int32), _ptr(weight, "weight", torch.float32),
-                                   T, E, int(top), int(bool(renorm)), ROUTER_SCORING[scoring], _stream()), "router_topk")
+                                   T, E, logits.shape[1], int(top), int(bool(renorm)), ROUTER_SCORING[scoring], count, keep, _stream()),
+           "router_topk")
 
 
-def moe_combine(y, weight, extra, out, T, top):
-    """out[t] = sum_j weight[t*top + j] * y[t*top + j] (+ extra[t]); all fp32; ``weight`` None: every weight 1."""
+def moe_combine(y, weight, extra, out, T, top, gate=None):
+    """out[t] = sum_j weight[t*top + j] * y[t*top + j] (+ extra[t]); all fp32; ``weight`` None: every weight 1.
+    ``gate`` (fp32, [T] with any stride): the extra row is multiplied by sigmoid(gate[t])."""
+    if gate is not None and (gate.dim() != 1 or gate.shape[0] < T or gate.dtype != torch.float32 or not gate.is_cuda or extra is None):
+        raise KernelError("moe_combine: a gate is one fp32 number a token for the extra row")
     d = out.shape[-1]
     if y.numel() < T * top * d or (weight is not None and weight.numel() < T * top) or out.numel() < T * d \
             or (extra is not None and extra.numel() < T * d):
         raise KernelError("moe_combine: arrays too small")
     _check(lib().spite_moe_combine(_ptr(y, "y", torch.float32), _ptr(weight, "weight", torch.float32, True),
-                                   _ptr(extra, "extra", torch.float32, True), _ptr(out, "out", torch.float32),
-                                   T, d, int(top), _stream()), "moe_combine")
+                                   _ptr(extra, "extra", torch.float32, True),
+                                   gate.data_ptr() if gate is not None else None, gate.stride(0) if gate is not None else 0,
+                                   _ptr(out, "out", torch.float32), T, d, int(top), _stream()), "moe_combine")
 
 
 def gated_rows(a, ids, table, col0, g):
@@ -799,7 +862,7 @@ def attn_latent_mfma(q, kv_pages, out, positions, seq_of_token, block_table, wg,
 def qkv_prepare(qkv, q_out, k_pages, v_pages, positions, slot_map, HQ, GK, GV, D, Vd, page_size, *, bias=None,
                 norm_q=None, norm_k=None, eps=0.0, inv_freq=None, rot=0, inv_freq_v=None, write_kv=True,
                 k_tiled=False, v_tiled=False, stored_dim=None, rot_magnitude=1.0, head_norm=False, q_temperature=None,
-                values_from_keys=False):
+                values_from_keys=False, blend=None):
     """Between a fused projection and the cache (see attn_wide.hip).  qkv: rows that begin with
     [HQ*D | GK*D | GV*Vd] (further columns are left alone); ``bias`` fp32 over those; ``norm_q`` /
     ``norm_k`` (fp32 [HQ*D], [GK*D]): weights of an RMS norm over the whole q and the whole k part;
@@ -811,7 +874,12 @@ def qkv_prepare(qkv, q_out, k_pages, v_pages, positions, slot_map, HQ, GK, GV, D
     ``head_norm``: ``norm_q`` / ``norm_k`` hold D weights each and every head is normed on its own.
     ``q_temperature`` = (coef, every): the queries (after their norm) times 1 + coef * ln(floor((p + 1) / every) + 1)
     at position p.  ``values_from_keys``: the row holds no values, [HQ*D | GK*D] only; the values are the keys as
-    the row holds them, before norm and rotation (GV = GK, Vd = D)."""
+    the row holds them, before norm and rotation (GV = GK, Vd = D).  ``blend`` = (other [T, >= GV*Vd] in the rows'
+    dtype, rows may lie apart; lam): the cached values are (1 - lam) v + lam other."""
+    other, lam = blend if blend is not None else (None, 0.0)
+    if other is not None and (other.dim() != 2 or other.stride(1) != 1 or other.shape[1] < GV * Vd or other.shape[0] < qkv.shape[0]
+                              or other.dtype != qkv.dtype or not other.is_cuda):
+        raise KernelError(f"qkv_prepare: values {tuple(other.shape)} {other.dtype} to blend with {GV} heads of {Vd}")
     T = qkv.shape[0]
     Dp = int(stored_dim or D)
     n = (HQ + GK) * D + (0 if values_from_keys else GV * Vd)
@@ -845,16 +913,19 @@ def qkv_prepare(qkv, q_out, k_pages, v_pages, positions, slot_map, HQ, GK, GV, D
         _ptr(inv_freq, "inv_freq", torch.float32, True), int(rot), float(rot_magnitude),
         _ptr(inv_freq_v, "inv_freq_v", torch.float32, True),
         T, HQ, GK, GV, D, Vd, page_size, int(bool(k_tiled)), int(bool(v_tiled)), Dp, int(bool(head_norm)), qt_coef, qt_every,
-        int(bool(values_from_keys)), _stream()), "qkv_prepare")
+        int(bool(values_from_keys)), other.data_ptr() if other is not None else None, other.stride(0) if other is not None else 0,
+        float(lam), _stream()), "qkv_prepare")
 
 
 def attn_wide(q, k_pages, v_pages, out, positions, seq_of_token, block_table, T, HQ, GK, GV, D, Vd, page_size, vis, span,
-              scale, k_tiled=False, v_tiled=False, sinks=None, slopes=None):
+              scale, k_tiled=False, v_tiled=False, sinks=None, slopes=None, keep=0, dist_bias=None):
     """Attention over the paged cache with keys of D and values of Vd elements, HQ query heads over
     GK key heads over GV value heads (query head h: key head h // (HQ/GK), value head of that % GV);
     any mix of portions and single tokens.  q [T, HQ*D]; out [T, HQ*Vd] in q's dtype or fp32.
     ``sinks`` (fp32 [HQ] or None): one more term exp(sinks[h]) in every softmax's denominator.
-    ``slopes`` (fp32 [HQ] or None): slopes[h] * (key position - query position) is added to the scaled score."""
+    ``slopes`` (fp32 [HQ] or None): slopes[h] * (key position - query position) is added to the scaled score.
+    ``keep``: with a chunk or a window the request's first so many keys are read too.  ``dist_bias`` (fp32 [HQ, n] or
+    None): dist_bias[h, min(p - j, n - 1)] is added to the scaled score."""
     if sinks is not None and sinks.numel() != HQ:
         raise KernelError(f"attention: {sinks.numel()} sinks for {HQ} query heads")
     if q.numel() < T * HQ * D or out.numel() < T * HQ * Vd:
@@ -871,7 +942,8 @@ def attn_wide(q, k_pages, v_pages, out, positions, seq_of_token, block_table, T,
         dtype_code(out.dtype), _ptr(positions, "positions", torch.int32), _ptr(seq_of_token, "seq_of_token", torch.int32),
         _ptr(block_table, "block_table", torch.int32), block_table.shape[1], T, HQ, GK, GV, D, Vd, page_size,
         VIS[vis], int(span or 0), float(scale), int(bool(k_tiled)), int(bool(v_tiled)),
-        _ptr(sinks, "sinks", torch.float32, True), _slopes(slopes, HQ), _stream()), "attention")
+        _ptr(sinks, "sinks", torch.float32, True), _slopes(slopes, HQ), int(keep), *_dist_bias(dist_bias, HQ), _stream()),
+        "attention")
 
 
 def attn_finish(a, out, positions, H, Vd, *, maps=1, lam=0.0, eps=0.0, post=1.0, inv_freq_v=None, gate=None):

@@ -13,6 +13,7 @@ CacheManager::CacheManager(int page_size, int max_requests, const std::vector<Gr
         if (g.n_pages < 1) throw std::invalid_argument("every group needs at least one page");
         if (g.kind < 0 || g.kind >= SP_VIS_COUNT) throw std::invalid_argument("unknown visibility");
         if (sp_vis_has_span(g.kind) && g.span < 1) throw std::invalid_argument("chunk or window must be >= 1");
+        if (g.keep < 0) throw std::invalid_argument("a group cannot keep fewer than no positions");
     }
     free_.resize(groups_.size());
     for (size_t g = 0; g < groups_.size(); ++g) {
@@ -120,7 +121,9 @@ int CacheManager::commit(int slot, int64_t n) {
     for (int g = 0; g < n_groups(); ++g) {
         const int64_t frontier = first_visible(sl.cached, groups_[g].kind, groups_[g].span);
         const int64_t upto = std::min<int64_t>(frontier / page_size_, (int64_t)sl.table[g].size());
-        for (int64_t b = sl.freed_below[g]; b < upto; ++b) {
+        // pages that hold one of the kept first positions stay
+        const int64_t kept = ((int64_t)groups_[g].keep + page_size_ - 1) / page_size_;
+        for (int64_t b = std::max(sl.freed_below[g], kept); b < upto; ++b) {
             int& page = sl.table[g][b];
             if (page >= 0) { free_[g].push_back(page); page = -1; }
         }
@@ -157,6 +160,7 @@ int64_t CacheManager::peak_pages(int64_t total, int64_t portion, int g) const {
     int64_t worst;
     if (groups_[g].kind == SP_VIS_CHUNK && groups_[g].span % ps == 0) worst = (back + n + ps - 1) / ps;
     else worst = (back + n - 1) / ps + 2;
+    worst += (groups_[g].keep + ps - 1) / ps;
     return std::min(all, worst);
 }
 

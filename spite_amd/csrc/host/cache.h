@@ -2,7 +2,8 @@
 // group of layers, and slots for per-request state of fixed size.
 //
 // A group is a set of layers with the same need: every key (full), the keys of the chunk
-// that the query lies in (chunk, size C), or the last W keys (window).  Each group has a
+// that the query lies in (chunk, size C), or the last W keys (window); with the two latter a
+// request's first positions may be kept in sight for good (keep).  Each group has a
 // pool of pages of its own.  A page holds `page_size` consecutive positions of one request
 // for all layers of the group.  The free list is a stack, as in the reference's BlockPool
 // (crates/spite-kvcache/src/paged.rs:55,89-93), so a page that is given back is the next one
@@ -27,6 +28,7 @@ struct GroupSpec {
     int kind;      // Visibility
     int span;      // chunk size or window; unused for full
     int n_pages;   // pool size
+    int keep = 0;  // first positions of a request that every later query reads (chunk, window): never given back
 };
 
 // First position that a query at position p may read: the rule shared with the attention kernels.

@@ -20,10 +20,10 @@ int spite_host_abi_version() { return 1; }
 
 // ---------------------------------------------------------------- cache manager
 void* spc_create(int page_size, int max_requests, int n_groups, const int* kinds, const int* spans,
-                 const int* n_pages) {
+                 const int* n_pages, const int* keeps) {
     SP_TRY
     std::vector<GroupSpec> gs;
-    for (int i = 0; i < n_groups; ++i) gs.push_back(GroupSpec{kinds[i], spans[i], n_pages[i]});
+    for (int i = 0; i < n_groups; ++i) gs.push_back(GroupSpec{kinds[i], spans[i], n_pages[i], keeps ? keeps[i] : 0});
     return (void*)new CacheManager(page_size, max_requests, gs);
     SP_CATCH(nullptr)
 }

@@ -18,7 +18,7 @@ def lib():
         l.spite_host_last_error.restype = c_char_p
         P, I, LL, ULL = c_void_p, c_int, c_longlong, c_ulonglong
         sigs = {
-            "spc_create": (P, [I, I, I, PI, PI, PI]),
+            "spc_create": (P, [I, I, I, PI, PI, PI, PI]),
             "spc_destroy": (None, [P]),
             "spc_admit": (I, [P]),
             "spc_take_fresh": (I, [P, PI, I]),

@@ -4,7 +4,8 @@
 // reads the names, in the order of their codes, from either library.
 //
 // A rule is "the query at position p reads the keys first_visible(p) .. p".  A new rule is a
-// new code, its name, and its case in sp_first_visible.
+// new code, its name, and its case in sp_first_visible.  Beside the rule a number `keep` may stand: the
+// request's first `keep` positions stay in sight of every later query, however far away (sp_visible).
 //
 // The includer defines SP_VIS_FN (the function qualifiers of its compiler) before including.
 #pragma once
@@ -26,3 +27,8 @@ SP_VIS_FN I sp_first_visible(I p, int vis, int span) {
     if (vis == SP_VIS_WINDOW) return p - span + 1 > 0 ? p - span + 1 : 0;
     return 0;
 }
+
+// Whether the query at p, whose rule starts at `first` (sp_first_visible), reads the key at j when the
+// request's first `keep` positions stay in sight.
+template <typename I>
+SP_VIS_FN bool sp_visible(I j, I p, I first, I keep) { return j <= p && (j >= first || j < keep); }

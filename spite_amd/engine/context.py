@@ -101,6 +101,7 @@ class StepContext:
     n_out: int
     host: HostBatch
     ws: Any = None               # Workspace of the layer call that runs
+    step_ws: Any = None          # Workspace whose memory lives as long as the step
     decode_only: bool = False    # every entry holds one token
     max_count: int = 0           # longest portion of the step
     derived: dict = field(default_factory=dict)   # step arrays that parts asked for: name -> (device array, info)

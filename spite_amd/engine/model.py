@@ -125,6 +125,7 @@ class Model:
         that the next norm has to add (``pending``), what a block's stages hand each other and,
         after the tail, ``logits``."""
         n, d = len(self.spec.order), self.spec.hidden_size
+        ctx.step_ws = step_ws
         for u in range(lo, hi):
             kind, _, i, stage = self._units[u]
             if kind == "embed":

@@ -39,6 +39,8 @@ class KVNeed:
     v_head_dim: Optional[int] = None  # width of a value where it differs from a key's (the pool's two halves are sized apart)
     n_v_heads: Optional[int] = None   # value heads where they are fewer than the key heads (several key heads, the
                                       # score maps of one head, share a value head)
+    keep: int = 0                     # with a chunk or a window: the request's first positions that every later query
+                                      # reads as well, however far away
 
     @property
     def value_dim(self) -> int:
@@ -164,12 +166,21 @@ class PositionEncoding(Part):
         a cap, if there is one), or None.  The attention kernels take it as an option."""
         return None
 
+    def score_table(self, n_heads: int):
+        """For encodings that bias the scores by distance: an fp32 tensor [n_heads, n] on the GPU, after loading; head
+        h's score of (query at p, key at j) gets table[h, min(p - j, n - 1)] added, or None."""
+        return None
+
     def transform(self, qkv, positions, n_heads, n_kv_heads, head_dim) -> None:
         """For encodings the fused kernel does not know: change q and k of the fused
         projection's rows in place before they are normed and cached."""
 
 
 class Mixer(Part):
+    """What a mixer leaves for later layers of the same step (a tensor taken from ``ctx.step_ws``, which lives as long as
+    the step) it puts under a name into ``ctx.extras["carried"]``, a dict that blocks hand from mixer to mixer through
+    the step's state (``run_mixer`` in block.py)."""
+
     def cache_need(self) -> CacheNeed:
         return CacheNeed()
 

@@ -9,18 +9,37 @@ import torch
 from .base import Block, NormedIncrement, NORMED_INCREMENTS, register, build as build_part, two_increments
 
 
+CARRY = "carried:"
+
+
+def run_mixer(mixer, x, state, ctx, cache):
+    """The mixer's forward with what earlier mixers of the step left for later ones under ``ctx.extras["carried"]``;
+    what this one leaves there goes into the step's state (every entry a key of its own, so that a captured step
+    knows the addresses)."""
+    had = {k[len(CARRY):]: v for k, v in state.items() if k.startswith(CARRY)}
+    ctx.extras["carried"] = carried = dict(had)
+    out = mixer.forward(x, ctx, cache)
+    for name, t in carried.items():
+        if had.get(name) is not t:
+            state[CARRY + name] = t
+    return out
+
+
 @register("block", "prenorm")
 class PreNormBlock(Block):
+    """The feed-forward (and its norm) may be missing."""
     graph_safe = True
 
     def __init__(self, env, spec):
         self.env = env
         self.norm1 = build_part("norm", spec.norm1, env)
         self.mixer = build_part("mixer", spec.mixer, env)
-        self.norm2 = build_part("norm", spec.norm2, env)
-        self.ffn = build_part("ffn", spec.ffn, env)
-        self.children = (("norm1", self.norm1, spec.norm1), ("mixer", self.mixer, spec.mixer),
-                         ("norm2", self.norm2, spec.norm2), ("ffn", self.ffn, spec.ffn))
+        self.children = (("norm1", self.norm1, spec.norm1), ("mixer", self.mixer, spec.mixer))
+        self.norm2 = self.ffn = None
+        if spec.ffn is not None:
+            self.norm2 = build_part("norm", spec.norm2, env)
+            self.ffn = build_part("ffn", spec.ffn, env)
+            self.children += (("norm2", self.norm2, spec.norm2), ("ffn", self.ffn, spec.ffn))
         self.graph_safe = all(part.graph_safe for _, part, _ in self.children)
         self.step_arrays = tuple(sorted({a for _, part, _ in self.children for a in part.step_arrays}))
 
@@ -33,8 +52,8 @@ class PreNormBlock(Block):
     def stages(self):
         # first norm | mixer | second norm and feed-forward: a mixer that reads the step's metadata
         # on the host keeps only itself out of a graph
-        return [(self.norm1.graph_safe, self._stage_norm1), (self.mixer.graph_safe, self._stage_mixer),
-                (self.norm2.graph_safe and self.ffn.graph_safe, self._stage_ffn)]
+        rest = self.ffn is None or (self.norm2.graph_safe and self.ffn.graph_safe)
+        return [(self.norm1.graph_safe, self._stage_norm1), (self.mixer.graph_safe, self._stage_mixer), (rest, self._stage_ffn)]
 
     def _stage_norm1(self, state, ctx, cache):
         h = state["h"]
@@ -44,10 +63,13 @@ class PreNormBlock(Block):
         state["normed"] = n
 
     def _stage_mixer(self, state, ctx, cache):
-        state["mixed"] = self.mixer.forward(state.pop("normed"), ctx, cache)
+        state["mixed"] = run_mixer(self.mixer, state.pop("normed"), state, ctx, cache)
 
     def _stage_ffn(self, state, ctx, cache):
         h, delta, ws = state["h"], state.pop("mixed"), ctx.ws
+        if self.ffn is None:
+            state["pending"] = (delta,)
+            return
         T, d = h.shape
         n2 = ws.take((T, d), self.env.dtype)
         proj = self.ffn.input_projection()
@@ -130,7 +152,7 @@ class SandwichBlock(Block):
         state["normed"] = n
 
     def _stage_mixer(self, state, ctx, cache):
-        state["mixed"] = self.mixer.forward(state.pop("normed"), ctx, cache)
+        state["mixed"] = run_mixer(self.mixer, state.pop("normed"), state, ctx, cache)
 
     def _stage_rest(self, state, ctx, cache):
         h, ws = state["h"], ctx.ws
@@ -266,7 +288,7 @@ class ParallelBlock(Block):
         state["ffn_in"] = (n, n32 if self.ffn.wants_f32_input and logits is None else None, logits)
 
     def _stage_mixer(self, state, ctx, cache):
-        state["mixed"] = self.mixer.forward(state.pop("mixer_in"), ctx, cache["mixer"] if isinstance(cache, dict) else cache)
+        state["mixed"] = run_mixer(self.mixer, state.pop("mixer_in"), state, ctx, cache["mixer"] if isinstance(cache, dict) else cache)
 
     def _stage_ffn(self, state, ctx, cache):
         pend = (state.pop("mixed"),)

@@ -24,6 +24,13 @@ gets an output row of its own and a last kernel forms the weighted sum per token
 With ``weight_input`` the weight multiplies the expert's input instead (the grouped product scales the rows it
 reads) and the outputs are summed as they are.
 
+``scoring="softmax"``: s = softmax over all experts.  ``groups`` = (count, keep): the experts form equal groups of
+neighbours and a token takes experts of its ``keep`` best groups only (a group's value: its largest s + bias).
+``shared_gate``: the shared expert's result times sigmoid of one number a token, a row of its own beside the
+router's (``shared.sg``), formed with the router's logits.  Experts and shared expert may have a gated activation
+with a bound of their own each (``activation="clamped"``, ``limit``, ``shared_limit``; so may ``dense_glu``):
+min(g, L) sigmoid(1.702 min(g, L)) (clamp(u, -L, L) + 1).
+
 ``moe_topk_softmax``: the same part with the other way of scoring: the ``top_k`` experts with the largest
 logits are taken and their weights are the softmax over the taken logits alone; no bias.
 """
@@ -38,16 +45,23 @@ from .linear import SKINNY_MAX_ROWS, Weight, grouped_tile_shape, linear
 from ..csrc import hipops
 
 
+def gate_activation(what, activation, limit):
+    """What ``linear`` takes as ``glu``: the activation's name, with its bound where it has one."""
+    if not isinstance(activation, str) or hipops.GATE_ACTS.get(activation, 0) == 0:
+        raise ValueError(f"{what}: activation {activation!r} (known: silu, gelu_tanh, relu, clamped)")
+    if (activation == "clamped") != (limit is not None) or (limit is not None and not float(limit) > 0.0):
+        raise ValueError(f"{what}: activation {activation!r} with the bound {limit!r} (clamped takes one above 0, the others none)")
+    return activation if limit is None else (activation, float(limit))
+
+
 @register("ffn", "dense_glu")
 class DenseGLU(FeedForward):
     graph_safe = True
 
-    def __init__(self, env, hidden_size, intermediate_size, activation="silu"):
-        """``activation``: the gate's, ``silu``, ``gelu_tanh`` or ``relu``."""
+    def __init__(self, env, hidden_size, intermediate_size, activation="silu", limit=None):
+        """``activation``: the gate's, ``silu``, ``gelu_tanh``, ``relu`` or, with the bound ``limit``, ``clamped``."""
         self.d, self.F = int(hidden_size), int(intermediate_size)
-        if hipops.GATE_ACTS.get(activation, 0) == 0:
-            raise ValueError(f"dense_glu: activation {activation!r} (known: silu, gelu_tanh, relu)")
-        self.activation = activation
+        self.activation = gate_activation("dense_glu", activation, limit)
         self.w_gate_up = self.w_down = None
 
     def params(self):
@@ -219,9 +233,11 @@ class MoeTopKSigmoid(FeedForward):
     wants_f32_input = True
 
     def __init__(self, env, hidden_size, intermediate_size, n_experts, top_k, shared_intermediate_size=None,
-                 score_bias=True, renormalize=False, activation="silu", scoring="sigmoid", weight_input=False):
-        """``scoring``: ``sigmoid`` (the choice by sigmoid(z) + bias, weights sigmoid(z)) or ``softmax_taken`` (the
-        choice by z + bias, weights the softmax over the taken experts' z).  ``weight_input``: the weight multiplies
+                 score_bias=True, renormalize=False, activation="silu", scoring="sigmoid", weight_input=False, groups=None,
+                 shared_gate=False, limit=None, shared_limit=None):
+        """``scoring``: ``sigmoid`` (the choice by sigmoid(z) + bias, weights sigmoid(z)), ``softmax`` (the same with the
+        softmax over all experts) or ``softmax_taken`` (the choice by z + bias, weights the softmax over the taken
+        experts' z).  ``groups``: (count, keep); ``shared_gate``, ``limit``, ``shared_limit``: see above.  ``weight_input``: the weight multiplies
         the expert's input instead of its output: the result is the sum of expert(w * x)."""
         self.weight_input = bool(weight_input)
         if scoring not in hipops.ROUTER_SCORING:
@@ -231,9 +247,18 @@ class MoeTopKSigmoid(FeedForward):
         self.Fs = None if shared_intermediate_size is None else int(shared_intermediate_size)
         if not 1 <= self.k <= self.E or self.E > 512:
             raise ValueError(f"moe: {self.k} of {self.E} experts (at most 512)")
-        if hipops.GATE_ACTS.get(activation, 0) == 0:
-            raise ValueError(f"moe: activation {activation!r} (known: silu, gelu_tanh, relu)")
-        self.score_bias, self.renormalize, self.activation = bool(score_bias), bool(renormalize), activation
+        self.activation = gate_activation("moe", activation, limit)
+        self.shared_activation = None if self.Fs is None else \
+            gate_activation("moe: shared expert", activation, shared_limit if shared_limit is not None else limit)
+        self.score_bias, self.renormalize = bool(score_bias), bool(renormalize)
+        self.groups = None if groups is None else (int(groups[0]), int(groups[1]))
+        if self.groups is not None:
+            count, keep = self.groups
+            if count < 1 or self.E % count or not 1 <= keep <= count or self.k > keep * (self.E // count):
+                raise ValueError(f"moe: {self.k} experts out of {keep} of {count} groups of {self.E} experts")
+        self.shared_gate = bool(shared_gate)
+        if self.shared_gate and self.Fs is None:
+            raise ValueError("moe: a gate on a shared expert that there is not")
         self.w_router = self.bias = self.w_gate_up = self.w_down = self.ws_gate_up = self.ws_down = None
 
     def params(self):
@@ -246,11 +271,16 @@ class MoeTopKSigmoid(FeedForward):
         if self.Fs is not None:
             p["shared.gate"], p["shared.up"] = ParamSpec((self.Fs, d)), ParamSpec((self.Fs, d))
             p["shared.down"] = ParamSpec((d, self.Fs))
+        if self.shared_gate:
+            p["shared.sg"] = ParamSpec((1, d), kind="vector", init="normal")
         return p
 
     def load(self, t):
         E = self.E
         self.w_router = t["router"].contiguous()
+        if self.shared_gate:
+            # one more row: its product comes with the router's logits
+            self.w_router = torch.cat([self.w_router, t["shared.sg"]], dim=0).contiguous()
         self.bias = t["correction"].contiguous() if self.score_bias else None
         dts = {t[f"e{e}.{k}"].dtype for e in range(E) for k in ("gate", "up", "down")}
         dt = torch.float32 if len(dts) > 1 else dts.pop()
@@ -276,19 +306,24 @@ class MoeTopKSigmoid(FeedForward):
         ws = ctx.ws
         logits = projected
         if logits is None:
-            logits = ws.take((T, E), torch.float32)
-            hipops.gemm_generic(x32, self.w_router, logits, T, E, d)
+            P = self.w_router.shape[0]
+            logits = ws.take((T, P), torch.float32)
+            hipops.gemm_generic(x32, self.w_router, logits, T, P, d)
+        gate = logits[:, E] if self.shared_gate else None
         n = T * k
         expert, weight = ws.take((n,), torch.int32), ws.take((n,), torch.float32)
         trace = ctx.extras.get("trace")
-        bias = self.bias
+        bias, groups = self.bias, self.groups
         if trace is not None and trace.get("take_experts"):
             # a testing aid: the experts are given ([T, top_k] per call, in the order of the calls), each
             # with the weight that its own logit gives; every other logit is taken out of the choice
             take = trace["take_experts"].pop(0).to(device=x.device, dtype=torch.int64).view(T, k)
+            if self.scoring == "softmax" and not self.renormalize:
+                raise ValueError("moe: given experts under a softmax over all of them need renormalized weights")
             logits = torch.full_like(logits, float("-inf")).scatter_(1, take, logits.gather(1, take))
-            bias = None
-        hipops.router_topk(logits, bias, expert, weight, k, renorm=self.renormalize, scoring=self.scoring)
+            bias = groups = None
+        hipops.router_topk(logits, bias, expert, weight, k, renorm=self.renormalize, scoring=self.scoring, groups=groups,
+                           n_experts=E)
         if trace is not None:                         # a testing aid: which experts each token took, [T, top_k]
             trace.setdefault("moe_experts", []).append(expert.view(T, k).clone())
         # (``unused``: the entries' weights in the order of the slots; a product reads it only with ``weight_input``)
@@ -305,11 +340,11 @@ class MoeTopKSigmoid(FeedForward):
         ys = None
         if self.Fs is not None:
             act_s = ws.take((T, self.Fs), x.dtype)
-            linear(x, self.ws_gate_up, act_s, glu=self.activation, ws=ws)
+            linear(x, self.ws_gate_up, act_s, glu=self.shared_activation, ws=ws)
             ys = ws.take((T, d), torch.float32)
             linear(act_s, self.ws_down, ys, ws=ws)
         out = ws.take((T, d), torch.float32)
-        hipops.moe_combine(y, None if self.weight_input else weight, ys, out, T, k)
+        hipops.moe_combine(y, None if self.weight_input else weight, ys, out, T, k, gate=gate)
         return (out,)
 
 

@@ -12,6 +12,10 @@ so the attention kernel sees one shared kv head whose rows are ``kv_rank + rot_d
 value is the row's first ``kv_rank`` elements.  The two per-head products run as grouped products
 with one group a head over a row list (rows lie token by token, groups want them head by head).
 
+The queries may go through a latent of their own (``q_rank``): c_q = rmsnorm(W_dq x) with a weight, q = W_uq c_q; its
+down-projection is then one product with the cached latent's.  Without a rotated part (``rot_dim`` 0) there is no
+position encoding at all.
+
 A layer may read the rows that an earlier layer cached (``own_kv=False``): it has no
 down-projection, but queries, per-head matrices, mask and output projection of its own.
 """
@@ -37,12 +41,12 @@ class LatentAttention(Mixer):
     graph_safe = True
 
     def __init__(self, env, hidden_size, n_heads, dim, rot_dim, v_dim, kv_rank, scale, position, norm_eps,
-                 visibility="full", span=0, own_kv=True, cache_visibility=None, cache_span=None):
+                 visibility="full", span=0, own_kv=True, cache_visibility=None, cache_span=None, q_rank=None):
         """``dim`` / ``rot_dim``: unrotated / rotated query and key elements of a head; ``v_dim``: a head's
         value; ``kv_rank``: the latent.  ``position``: the encoding of the rotated parts (its frequency
-        table; adjacent pairs).  ``visibility`` / ``span``: what this layer's queries read;
+        table; adjacent pairs), None without them.  ``visibility`` / ``span``: what this layer's queries read;
         ``cache_visibility`` / ``cache_span``: what the cache must keep (the widest of all layers that
-        read it; default: this layer's own)."""
+        read it; default: this layer's own).  ``q_rank``: the queries' latent, if they have one."""
         if visibility not in hipops.VIS:
             raise ValueError(f"latent attention: visibility {visibility!r} (known: {sorted(hipops.VIS)})")
         if visibility != "full" and span < 1:
@@ -56,25 +60,31 @@ class LatentAttention(Mixer):
         self.cache_visibility = cache_visibility or visibility
         self.cache_span = int(cache_span if cache_span is not None else self.span)
         self.own = bool(own_kv)
-        self.position = build_part("position", position, env)
-        if self.position.kernel_args().get("magnitude", 1.0) != 1.0:
+        self.q_rank = int(q_rank or 0)
+        if position is None and self.r:
+            raise ValueError("latent attention: rotated parts without a position encoding")
+        self.position = build_part("position", position, env) if position is not None else None
+        ka = self.position.kernel_args() if self.position is not None else {"inv_freq": None}
+        if ka.get("magnitude", 1.0) != 1.0:
             raise ValueError("latent_attention: a position encoding that scales sine and cosine is not what this mixer's kernel applies")
-        ka = self.position.kernel_args()
         if self.r and not (ka.get("use_rope") and ka.get("adjacent")):
             raise ValueError("latent attention: the rotated parts take a rotary encoding with adjacent pairs")
         self.inv_freq = ka["inv_freq"]
         self.rot_dims = int(ka.get("rotary_dim") or 0)
         if self.rot_dims > self.r:
             raise ValueError(f"latent attention: {self.rot_dims} turning elements of a rotated part of {self.r}")
-        self.wq = self.wdkv = self.w_norm = self.w_absorb = self.w_up = self.wo = None
+        self.wq = self.wdkv = self.w_norm = self.wdq = self.w_qnorm = self.w_absorb = self.w_up = self.wo = None
         self.mfma = env.dtype == torch.bfloat16 and hipops.attn_latent_mfma_ok(self.Dk, self.R, 0)
         self._wg = _workgroups_name(self.H) if self.mfma else None
         self.step_arrays = (self._wg,) if self.mfma else ()
 
     def params(self):
         d, H, n, r, v, R = self.d, self.H, self.n, self.r, self.v, self.R
-        p = {"q": ParamSpec((H * (n + r), d)), "uk": ParamSpec((H * n, R)), "uv": ParamSpec((H * v, R)),
+        p = {"q": ParamSpec((H * (n + r), self.q_rank or d)), "uk": ParamSpec((H * n, R)), "uv": ParamSpec((H * v, R)),
              "o": ParamSpec((d, H * v))}
+        if self.q_rank:
+            p["dq"] = ParamSpec((self.q_rank, d))
+            p["dq.norm"] = ParamSpec((self.q_rank,), kind="vector", init="ones")
         if self.own:
             p["dkv"] = ParamSpec((R + r, d))
             p["dkv.norm"] = ParamSpec((R,), kind="vector", init="ones")
@@ -84,8 +94,14 @@ class LatentAttention(Mixer):
         H, n, v, R = self.H, self.n, self.v, self.R
         self.wq = Weight(t["q"])
         if self.own:
-            self.wdkv = Weight(t["dkv"])
             self.w_norm = t["dkv.norm"].contiguous()
+        if self.q_rank:
+            self.w_qnorm = t["dq.norm"].contiguous()
+        # the down-projections of both latents read the same rows: one product
+        down = [t[k] for k in ("dq", "dkv") if k in t]
+        if down:
+            dt = down[0].dtype if len({w.dtype for w in down}) == 1 else torch.float32
+            self.wdkv = Weight(torch.cat([w.to(dt) for w in down], dim=0))
         # U_h^T as a product's weight [out = R, in = n]; V_h is one already: [out = v, in = R]
         # (its input rows are column ranges of the query rows: operand order only if those stay aligned)
         self.w_absorb = Weight(t["uk"].view(H, n, R).transpose(1, 2).contiguous(), (n + self.r) % 8 == 0)
@@ -98,7 +114,7 @@ class LatentAttention(Mixer):
             if not hipops.attn_latent_mfma_ok(self.Dk, self.R, page_size):
                 notes.append(f"latent attention runs on plain FMAs: rows of {self.Dk} with a latent of {self.R} "
                              f"(the MFMA kernel takes multiples of 8, rows up to 576, latents up to 512)")
-            for name, w in (("query projection", self.wq), ("down-projection", self.wdkv), ("per-head key matrices", self.w_absorb),
+            for name, w in (("query projection", self.wq), ("down-projections", self.wdkv), ("per-head key matrices", self.w_absorb),
                             ("per-head value matrices", self.w_up), ("output projection", self.wo)):
                 if w is not None:
                     notes += w.slow_reason(name)
@@ -114,18 +130,30 @@ class LatentAttention(Mixer):
         T = x.shape[0]
         H, n, r, v, R, Dk = self.H, self.n, self.r, self.v, self.R, self.Dk
         ws = ctx.ws
+        Q = self.q_rank
         q = ws.take((T, H * (n + r)), x.dtype)
-        linear(x, self.wq, q, ws=ws)
-        dkv = None
-        if self.own:
-            if not cache.write:
+        if not Q:
+            linear(x, self.wq, q, ws=ws)
+        down = dkv = latent = None
+        if self.wdkv is not None:
+            if self.own and not cache.write:
                 raise RuntimeError("latent attention: a layer with a down-projection of its own must write its cache")
-            dkv = ws.take((T, R + r), x.dtype)
-            linear(x, self.wdkv, dkv, ws=ws)
+            down = ws.take((T, self.wdkv.shape[0]), x.dtype)
+            linear(x, self.wdkv, down, ws=ws)
+        if self.own:
+            dkv = down[:, Q:]
+        if Q:
+            latent = (down, self.w_qnorm, ws.take((T, Q), x.dtype))
         qa = ws.take((T * H, Dk), x.dtype)
         rows_th, offsets_h = ws.take((H * T,), torch.int32), ws.take((H + 1,), torch.int32)
-        hipops.latent_prepare(q, dkv, qa, cache.k_pages, ctx.positions, cache.slot_map, self.inv_freq, self.w_norm,
-                              self.eps, H, n, r, R, self.rot_dims, self.own, rows_th, offsets_h)
+        prepare = lambda qd, own, query_latent: hipops.latent_prepare(
+            qd, dkv if own else None, qa, cache.k_pages, ctx.positions, cache.slot_map, self.inv_freq, self.w_norm,
+            self.eps, H, n, r, R, self.rot_dims, own, rows_th, offsets_h, query_latent=query_latent)
+        prepare(None if Q and self.own else q, self.own, latent)
+        if Q:
+            linear(latent[2], self.wq, q, ws=ws)
+            if r:
+                prepare(q, False, None)                 # the rotated parts of queries that came after their latent's norm
         # U_h^T a_h into the first R elements of every query row: one group a head
         linear(q.view(T * H, n + r)[:, :n], self.w_absorb, qa[:, :R], offsets=offsets_h, n_groups=H, a_rows=rows_th,
                y_rows=rows_th, rows=H * T, max_rows=T, ws=ws)

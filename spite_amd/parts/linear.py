@@ -108,7 +108,7 @@ def linear(x, w, y, *, glu=False, offsets=None, n_groups=1, a_rows=None, a_scale
     """y[r] = W . x[r] for ``rows`` rows (default: all of x; for a row list: its length).
 
     With ``glu`` the weight holds gate rows then up rows and y = act(gate) * up: ``True`` or
-    ``"silu"``, or ``"gelu_tanh"``.
+    ``"silu"``, ``"gelu_tanh"``, ``"relu"`` or ``("clamped", limit)`` (``hipops.gate_code``).
     ``max_rows``: the most rows that one group can bring (default: ``rows``).
     ``tile_shape``: the prefill product's tile (``grouped_tile_shape``), 0 = the library's choice.
     ``live_groups``: a promise that at most this many groups hold rows (0: none).
@@ -119,7 +119,7 @@ def linear(x, w, y, *, glu=False, offsets=None, n_groups=1, a_rows=None, a_scale
     tiled = False
     if isinstance(w, Weight):
         w, tiled = w.data, w.tiled
-    glu = hipops.GATE_ACTS[glu]          # True or "silu", "gelu_tanh": the gate's activation
+    glu, limit = hipops.gate_code(glu)   # the gate's activation and its bound
     K = x.shape[-1]
     N = y.shape[-1]
     M = rows if rows is not None else x.shape[0]
@@ -131,7 +131,7 @@ def linear(x, w, y, *, glu=False, offsets=None, n_groups=1, a_rows=None, a_scale
         if most <= SKINNY_MAX_ROWS and not (tiled and most > 32 and offsets is None and N >= 65536):
             hipops.gemm_skinny(x, w, y, M, N, K, offsets=offsets, n_groups=n_groups, a_rows=a_rows,
                                a_scale=a_scale, y_rows=y_rows, glu=glu, max_rows=most, tiled=tiled,
-                               live_groups=live_groups, act=act)
+                               live_groups=live_groups, act=act, act_limit=limit)
             return
         if tiled:
             plain = offsets is None and a_rows is None and a_scale is None and y_rows is None and not glu and tile_shape == 0 \
@@ -139,10 +139,10 @@ def linear(x, w, y, *, glu=False, offsets=None, n_groups=1, a_rows=None, a_scale
             runs = hipops.tiled_k_runs(M, N, K) if plain and M > 0 else 1
             part = _scratch(ws, (runs, M, N), torch.float32, x.device) if runs > 1 else None
             hipops.gemm_tiled(x, w, y, M, N, K, offsets=offsets, n_groups=n_groups, a_rows=a_rows, a_scale=a_scale,
-                              y_rows=y_rows, glu=glu, shape=tile_shape, part=part, act=act)
+                              y_rows=y_rows, glu=glu, shape=tile_shape, part=part, act=act, act_limit=limit)
             return
         hipops.gemm_mfma(x, w, y, M, N, K, offsets=offsets, n_groups=n_groups, a_rows=a_rows, a_scale=a_scale,
-                         y_rows=y_rows, glu=glu)
+                         y_rows=y_rows, glu=glu, act_limit=limit)
         _act_after(y, M, y_rows, act)
         return
     if tiled:
@@ -151,17 +151,17 @@ def linear(x, w, y, *, glu=False, offsets=None, n_groups=1, a_rows=None, a_scale
         x32 = _widen(x, ws)
         if y.dtype == torch.float32:
             hipops.gemm_generic(x32, w, y, M, N, K, offsets=offsets, n_groups=n_groups, a_rows=a_rows,
-                                a_scale=a_scale, y_rows=y_rows, glu=glu)
+                                a_scale=a_scale, y_rows=y_rows, glu=glu, act_limit=limit)
             _act_after(y, M, y_rows, act)
         else:
             y32 = _scratch(ws, y.shape, torch.float32, y.device)
             hipops.gemm_generic(x32, w, y32, M, N, K, offsets=offsets, n_groups=n_groups, a_rows=a_rows,
-                                a_scale=a_scale, y_rows=y_rows, glu=glu)
+                                a_scale=a_scale, y_rows=y_rows, glu=glu, act_limit=limit)
             _act_after(y32, M, y_rows, act)
             hipops.convert(y32, y)
         return
     hipops.gemm_generic(x, w, y, M, N, K, offsets=offsets, n_groups=n_groups, a_rows=a_rows, a_scale=a_scale,
-                        y_rows=y_rows, glu=glu)
+                        y_rows=y_rows, glu=glu, act_limit=limit)
     _act_after(y, M, y_rows, act)
 
 

@@ -15,16 +15,17 @@ from ..csrc import hipops
 class RMSNorm(Norm):
     graph_safe = True
 
-    def __init__(self, env, width: int, eps: float):
+    def __init__(self, env, width: int, eps: float, offset: float = 0.0):
+        """``offset``: what the checkpoint's weight is the distance from (1: a weight stored around zero)."""
         self.width = int(width)
-        self.eps = float(eps)
+        self.eps, self.offset = float(eps), float(offset)
         self.weight = None
 
     def params(self):
-        return {"weight": ParamSpec((self.width,), kind="vector", init="ones")}
+        return {"weight": ParamSpec((self.width,), kind="vector", init="normal" if self.offset else "ones")}
 
     def load(self, tensors):
-        self.weight = tensors["weight"]
+        self.weight = tensors["weight"] if self.offset == 0.0 else (tensors["weight"] + self.offset).contiguous()
 
     def as_increment(self, y, mult: float):
         """This norm as the last step of a sublayer's result y on its way into the stream."""

@@ -17,6 +17,11 @@ table is computed in float64 and stored as fp32; angle and rotation are fp32 in 
 slope_h * (i - j) with slope_h = 2^(-ratio (h + 1) / H), H the number of heads: the further a key, the less it counts,
 each head at its own rate.
 
+``distance_buckets``: nothing is done to q and k; head h's score of (query at i, key at j) gets rel[bucket(i - j), h]
+added, with a learned table rel of B rows (the checkpoint decides how many) and bucket(n) = n for n < B/2, else
+min(B - 1, B/2 + floor(ln(n / (B/2)) / ln(far / (B/2)) (B - B/2))): a row each for near distances, then rows that widen
+with the logarithm, the last one from ``far`` on.  The attention kernels read it as a table by distance.
+
 ``none``: no position information (NoPE layers).
 """
 from __future__ import annotations
@@ -25,7 +30,7 @@ import math
 
 import torch
 
-from .base import PositionEncoding, register
+from .base import ParamSpec, PositionEncoding, register
 
 
 def rotation_magnitude(scaling=None) -> float:
@@ -112,3 +117,41 @@ class DistanceSlopes(PositionEncoding):
     def score_slopes(self, n_heads: int):
         vals = [2.0 ** (-self.ratio * (h + 1) / n_heads) for h in range(n_heads)]
         return torch.tensor(vals, dtype=torch.float64).to(torch.float32).to(self.env.device)
+
+
+def distance_bucket(n: int, buckets: int, far: float) -> int:
+    """The row of a table of ``buckets`` rows that distance n reads."""
+    half = buckets // 2
+    if n < half:
+        return n
+    return min(buckets - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (buckets - half)))
+
+
+@register("position", "distance_buckets")
+class DistanceBuckets(PositionEncoding):
+    graph_safe = True
+
+    def __init__(self, env, n_heads: int, far: float, buckets: int = 32):
+        """``far``: the distance from which on every key reads the table's last row; ``buckets``: the rows that
+        random weights are drawn with (a checkpoint brings its own number)."""
+        self.env, self.H, self.far, self.buckets = env, int(n_heads), float(far), int(buckets)
+        self.table = None
+
+    def params(self):
+        return {"rel": ParamSpec((self.buckets, self.H), kind="vector", init="normal", free=(0,))}
+
+    def load(self, tensors):
+        rel = tensors["rel"]
+        B = rel.shape[0]
+        if B < 2 or not self.far > B // 2:
+            raise ValueError(f"distance_buckets: a table of {B} rows needs at least two, and a far distance above {B // 2} (it is {self.far})")
+        # by distance, up to the first one from which on every distance reads the last row
+        rows = [0]
+        while rows[-1] < B - 1:
+            rows.append(distance_bucket(len(rows), B, self.far))
+        self.table = rel.float()[torch.tensor(rows, device=rel.device)].t().contiguous()
+
+    def score_table(self, n_heads: int):
+        if n_heads != self.H:
+            raise ValueError(f"distance_buckets: a table for {self.H} heads met {n_heads}")
+        return self.table

@@ -29,7 +29,12 @@ keys and queries ``key_dim`` wide, values ``value_dim`` wide, with, each as an o
 * ``q_temperature`` = (coef, every): the normed queries at position p times 1 + coef ln(floor((p+1)/every) + 1);
 * ``values="keys"``: there is no value projection; the values are the keys as they leave the convolution,
   before their norm (``value_dim`` = ``key_dim``);
-* ``score_position``: a position part that works on the scores (per-head slopes on the distance).
+* ``score_position``: a position part that works on the scores (per-head slopes on the distance, or a learned bias by
+  distance, whose tensors are the mixer's under the part's own names);
+* ``keep``: beside a window or a chunk the request's first ``keep`` positions stay in sight of every later query;
+* ``value_blend``: the name under which the first layer of the step that has it leaves its values for the later ones,
+  which cache (1 - lambda) v + lambda v_first with a learned number lambda of their own (``v_mix``; the first layer's
+  is not used).
 
 Inside, two maps are 2H query heads over 2G key heads over G value heads: the projections' rows
 are reordered map by map when they are loaded, so that query head m*H + h reads key head
@@ -56,7 +61,7 @@ class WideAttention(Mixer):
     def __init__(self, env, hidden_size, n_heads, n_kv_heads, key_dim, value_dim, scale, position=None,
                  value_position=None, visibility="full", span=0, bias=False, projection_norm=False, norm_eps=1e-5,
                  maps=1, diff=0.0, head_gate=False, sinks=False, conv_taps=0, head_norm=False, q_temperature=None,
-                 values="projection", score_position=None):
+                 values="projection", score_position=None, keep=0, value_blend=None):
         if n_heads % n_kv_heads:
             raise ValueError(f"wide_attention: {n_heads} heads over {n_kv_heads} kv heads")
         if visibility not in hipops.VIS:
@@ -75,13 +80,19 @@ class WideAttention(Mixer):
             raise ValueError("wide_attention: a norm per head or one over the whole projection, not both")
         if (conv_taps or 0) >= 1 and (maps != 1 or bias or values != "keys"):
             raise ValueError("wide_attention: the convolution goes with one map, no biases and values taken from the keys")
+        if keep and (visibility == "full" or keep < 0):
+            raise ValueError(f"wide_attention: {keep} first positions kept beside {visibility!r} visibility")
+        if value_blend is not None and (values != "projection" or value_position is not None or bias):
+            raise ValueError("wide_attention: blended values come from a plain projection, without bias or rotation")
         if sinks not in (False, True, None, "zero"):
             raise ValueError(f"wide_attention: sinks {sinks!r} (known: True, 'zero')")
         self.env = env
         self.d, self.H, self.G = int(hidden_size), int(n_heads), int(n_kv_heads)
         self.D, self.Vd, self.maps = int(key_dim), int(value_dim), int(maps)
         self.scale, self.diff, self.eps = float(scale), float(diff), float(norm_eps)
-        self.visibility, self.span = visibility, int(span or 0)
+        self.visibility, self.span, self.keep = visibility, int(span or 0), int(keep or 0)
+        self.value_blend = value_blend
+        self.blend = 0.0
         self.bias, self.projection_norm, self.head_gate = bool(bias), bool(projection_norm), bool(head_gate)
         self.sinks = bool(sinks)
         self.zero_sinks = sinks == "zero"
@@ -92,18 +103,18 @@ class WideAttention(Mixer):
         if self.q_temperature is not None and self.q_temperature[1] < 1:
             raise ValueError(f"wide_attention: query temperature every {self.q_temperature[1]} positions")
         self.score_position = build_part("position", score_position, env) if score_position is not None else None
-        self.slopes = self.w_conv = None
+        self.slopes = self.dist_bias = self.w_conv = None
         self.position = build_part("position", position, env) if position is not None else None
         self.value_position = build_part("position", value_position, env) if value_position is not None else None
         for pe in (self.position, self.value_position):
             if pe is not None and (not pe.fused or pe.kernel_args().get("adjacent")):
                 raise ValueError("wide_attention: the position encoding must be a rotation in halves")
         self.HQ, self.GK = self.H * self.maps, self.G * self.maps
-        # the MFMA kernels take keys and values of one width, 64 or 128: narrower keys (and queries) are stored
-        # that wide in a bfloat16 run, zeros behind their own elements
-        self.Dk = self.D
-        if env.dtype == torch.bfloat16 and self.Vd in (64, 128) and self.D < self.Vd and self.HQ // self.GK <= 16:
-            self.Dk = self.Vd
+        # the MFMA kernels take certain pairs of key and value widths: narrower keys (and queries) are stored
+        # as wide as the next one in a bfloat16 run, zeros behind their own elements
+        wide = hipops.attn_stored_width(self.D, self.Vd)
+        self.mfma_widths = env.dtype == torch.bfloat16 and wide is not None and self.HQ // self.GK <= 16
+        self.Dk = wide if self.mfma_widths else self.D
         self.n_qk = (self.HQ + self.GK) * self.D
         self.n_qkv = self.n_qk + (0 if self.values_from_keys else self.G * self.Vd)
         self.w_in = self.wo = self.b_in = self.w_qnorm = self.w_knorm = None
@@ -134,6 +145,10 @@ class WideAttention(Mixer):
             p.update({k: ParamSpec((D,), kind="vector", init="normal") for k in ("lambda_q1", "lambda_k1", "lambda_q2", "lambda_k2")})
         if self.head_gate:
             p["gate_proj"] = ParamSpec((H, d))
+        if self.score_position is not None:
+            p.update(self.score_position.params())
+        if self.value_blend is not None:
+            p["v_mix"] = ParamSpec((), kind="vector", init="normal")
         if self.sinks and not self.zero_sinks:
             p["sink"] = ParamSpec((H,), kind="vector", init="normal")
         return p
@@ -167,7 +182,11 @@ class WideAttention(Mixer):
             # tap by tap, [taps, channels]: the kernel's loads of one tap are consecutive
             self.w_conv = torch.cat([t["q_conv"].float(), t["k_conv"].float()], dim=0).t().contiguous()
         if self.score_position is not None:
+            self.score_position.load({k: t[k] for k in self.score_position.params()})
             self.slopes = self.score_position.score_slopes(self.HQ)
+            self.dist_bias = self.score_position.score_table(self.HQ)
+        if self.value_blend is not None:
+            self.blend = float(t["v_mix"])
         if self.maps == 2:
             dot = lambda a, b: float((t[a].double() * t[b].double()).sum())
             self.lam = math.exp(dot("lambda_q1", "lambda_k1")) - math.exp(dot("lambda_q2", "lambda_k2")) + self.diff
@@ -192,8 +211,8 @@ class WideAttention(Mixer):
         if self.env.dtype == torch.bfloat16:
             if not self._mfma(page_size):
                 notes.append(f"attention runs on plain FMAs: keys of {self.D} and values of {self.Vd} elements, pages of "
-                             f"{page_size} (the MFMA kernels take values of 64 or 128 with keys no wider, at most 16 query heads "
-                             f"a kv head, and pages in multiples of 32)")
+                             f"{page_size} (the MFMA kernels take keys up to 64 with values of 32 or 64, keys up to 128 with values of "
+                             f"64 or 128, at most 16 query heads a kv head, and pages in multiples of 32)")
             for name, w in (("q/k/v projection", self.w_in), ("output projection", self.wo)):
                 if w is not None:
                     notes += w.slow_reason(name)
@@ -203,45 +222,55 @@ class WideAttention(Mixer):
         from .base import StateNeed
         # with a convolution: the last taps - 1 projected q and k rows of the request, fp32
         state = StateNeed((self.taps - 1, self.n_qk), torch.float32) if self.taps > 1 else None
-        return CacheNeed(kv=KVNeed(self.GK, self.Dk, self.visibility, self.span, v_head_dim=self.Vd, n_v_heads=self.G),
+        return CacheNeed(kv=KVNeed(self.GK, self.Dk, self.visibility, self.span, v_head_dim=self.Vd, n_v_heads=self.G, keep=self.keep),
                          state=state)
 
     def _mfma(self, page_size):
-        return (self.env.dtype == torch.bfloat16 and self.Dk == self.Vd and self.Vd in (64, 128) and page_size % 32 == 0
-                and self.HQ // self.GK <= 16)
+        return self.mfma_widths and page_size % 32 == 0
 
     # ------------------------------------------------------------------ the step
     def _decode(self, q, o, ctx, cache, T):
         HQ, GK, D = self.HQ, self.GK, self.Dk
         longest = cache.block_table.shape[1] * cache.page_size
         if self.visibility != "full":
-            longest = min(longest, self.span + 32)
+            longest = min(longest, self.span + self.keep + 32)
         blocks = -(-longest // 32)
         n_splits = max(1, min(-(-2 * hipops.cu_count() // (T * GK)), -(-blocks // 8), 256))
-        scratch = ctx.ws.take((hipops.attn_decode_workspace(T, HQ, D, n_splits) // 4,), torch.float32)
+        scratch = ctx.ws.take((hipops.attn_decode_workspace(T, HQ, self.Vd, n_splits) // 4,), torch.float32)
         hipops.attn_decode(q, cache.k_pages, cache.v_pages, o, scratch, ctx.positions, ctx.seq_of_token,
                            cache.block_table, T, HQ, GK, D, cache.page_size, self.visibility, self.span,
-                           self.scale, n_splits, value_heads=self.G, sinks=self.w_sink, slopes=self.slopes)
+                           self.scale, n_splits, value_heads=self.G, sinks=self.w_sink, slopes=self.slopes, v_dim=self.Vd,
+                           keep=self.keep, dist_bias=self.dist_bias)
 
     def _prefill(self, q, o, ctx, cache, lead, cu_seqlens):
         HQ, GK, D = self.HQ, self.GK, self.Dk
         counts, starts = ctx.host.counts[lead:], ctx.host.starts[lead:]
         longest = int((starts + counts).max())
         if self.visibility != "full":
-            longest = min(longest, self.span + int(counts.max()))
+            longest = min(longest, self.span + self.keep + int(counts.max()))
         n_splits = hipops.attn_prefill_splits(counts, HQ, GK, longest)
         scratch = None
         if n_splits > 1:
-            scratch = ctx.ws.take((hipops.attn_prefill_workspace(counts, HQ, GK, D, n_splits) // 4,), torch.float32)
+            scratch = ctx.ws.take((hipops.attn_prefill_workspace(counts, HQ, GK, self.Vd, n_splits) // 4,), torch.float32)
         hipops.attn_prefill(q, cache.k_pages, cache.v_pages, o, ctx.positions[lead:], cu_seqlens, counts,
                             cache.block_table[lead:], HQ, GK, D, cache.page_size, self.visibility, self.span, self.scale,
-                            n_splits=n_splits, scratch=scratch, value_heads=self.G, sinks=self.w_sink, slopes=self.slopes)
+                            n_splits=n_splits, scratch=scratch, value_heads=self.G, sinks=self.w_sink, slopes=self.slopes,
+                            v_dim=self.Vd, keep=self.keep, dist_bias=self.dist_bias)
 
     def forward(self, x, ctx, cache):
         T, ws = x.shape[0], ctx.ws
         H, G, HQ, GK, D, Vd, Dk = self.H, self.G, self.HQ, self.GK, self.D, self.Vd, self.Dk
-        proj = ws.take((T, self.n_in), x.dtype)
+        blend = leave = None
+        if self.value_blend is not None:
+            first = ctx.extras["carried"].get(self.value_blend)
+            if first is None:
+                leave = ctx.step_ws            # later layers of the step read this layer's values where the projection wrote them
+            else:
+                blend = (first, self.blend)
+        proj = (leave or ws).take((T, self.n_in), x.dtype)
         linear(x, self.w_in, proj, ws=ws)
+        if leave is not None:
+            ctx.extras["carried"][self.value_blend] = proj[:, self.n_qk:self.n_qk + self.G * Vd]
         conv = None
         if self.taps:
             # (with values taken from the keys the convolved rows are all that the next kernel reads)
@@ -253,7 +282,7 @@ class WideAttention(Mixer):
                            cache.page_size, bias=self.b_in, norm_q=self.w_qnorm, norm_k=self.w_knorm, eps=self.eps,
                            inv_freq=self.inv_freq, rot=self.rot, inv_freq_v=self.inv_freq_v, write_kv=cache.write,
                            k_tiled=cache.tiled, v_tiled=cache.tiled, stored_dim=Dk, rot_magnitude=self.rot_magnitude,
-                           head_norm=self.head_norm, q_temperature=self.q_temperature, values_from_keys=self.values_from_keys)
+                           head_norm=self.head_norm, q_temperature=self.q_temperature, values_from_keys=self.values_from_keys, blend=blend)
         if cache.tiled and self._mfma(cache.page_size):
             a = ws.take((T, HQ * Vd), x.dtype)
             cu_tail, lead = ctx.derived[TAIL]
@@ -268,7 +297,8 @@ class WideAttention(Mixer):
             a = ws.take((T, HQ * Vd), torch.float32 if self.maps == 2 else x.dtype)
             hipops.attn_wide(q, cache.k_pages, cache.v_pages, a, ctx.positions, ctx.seq_of_token, cache.block_table,
                              T, HQ, GK, G, Dk, Vd, cache.page_size, self.visibility, self.span, self.scale,
-                             k_tiled=cache.tiled, v_tiled=cache.tiled, sinks=self.w_sink, slopes=self.slopes)
+                             k_tiled=cache.tiled, v_tiled=cache.tiled, sinks=self.w_sink, slopes=self.slopes, keep=self.keep,
+                             dist_bias=self.dist_bias)
         if self.maps == 2 or self.inv_freq_v is not None or self.head_gate:
             o = ws.take((T, H * Vd), x.dtype)
             gate = proj[:, self.n_qkv:self.n_qkv + H] if self.head_gate else None

@@ -279,8 +279,11 @@ def test_the_visibility_rules_have_one_definition():
     codes = build.visibility_codes()
     assert codes == {"full": 0, "chunk": 1, "window": 2} and hipops.VIS == codes and paged._KINDS == codes
     lib = hostlib.lib()
-    for kind, span, n, first in (("full", 0, 37, 0), ("chunk", 8, 37, 32), ("window", 8, 37, 30), ("window", 8, 5, 0)):
-        h = lib.spc_create(4, 1, 1, hostlib.int_array([codes[kind]]), hostlib.int_array([span]), hostlib.int_array([32]))
+    for kind, span, n, first, keep in (("full", 0, 37, 0, 0), ("chunk", 8, 37, 32, 0), ("window", 8, 37, 30, 0), ("window", 8, 5, 0, 0),
+                                       ("window", 8, 37, 30, 1), ("window", 8, 37, 30, 4), ("window", 8, 37, 30, 5),
+                                       ("window", 8, 37, 30, 60), ("chunk", 8, 37, 32, 9)):
+        h = lib.spc_create(4, 1, 1, hostlib.int_array([codes[kind]]), hostlib.int_array([span]), hostlib.int_array([32]),
+                           hostlib.int_array([keep]))
         s = lib.spc_admit(h)
         assert lib.spc_reserve(h, s, n) == 0 and lib.spc_commit(h, s, n) == 0
         n_tab = lib.spc_table_len(h, s, 0)
@@ -288,5 +291,18 @@ def test_the_visibility_rules_have_one_definition():
         lib.spc_table(h, s, 0, tab, n_tab)
         held = [i for i in range(n_tab) if tab[i] >= 0]
         # the next query (position n) reads from `first`: pages wholly below it are gone
-        assert held == list(range(first // 4, -(-n // 4))), (kind, span, held)
+        # (but those that hold one of the kept first positions stay)
+        assert held == [b for b in range(-(-n // 4)) if b >= first // 4 or b * 4 < keep], (kind, span, keep, held)
+        if kind != "full":
+            lib.spc_release(h, s)
+            assert lib.spc_free_pages(h, 0) == 32 and lib.spc_check(h) == 0
+            # a portion of 4 positions after 96: no more pages than the manager promises, and all come back
+            s, most = lib.spc_admit(h), 0
+            for _ in range(25):
+                assert lib.spc_reserve(h, s, 4) == 0
+                most = max(most, 32 - lib.spc_free_pages(h, 0))
+                assert lib.spc_commit(h, s, 4) == 0 and lib.spc_check(h) == 0
+            assert most <= lib.spc_peak_pages(h, 100, 4, 0) <= 32
+            lib.spc_release(h, s)
+            assert lib.spc_free_pages(h, 0) == 32
         lib.spc_destroy(h)
