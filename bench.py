@@ -238,6 +238,13 @@ class KernelTimes:
 # attention with learned sinks and 64 turning elements beside time mixing with heads of 128), tanh norms before and
 # after every sublayer, the first two layers behind a reentry product (a loop walked once), the hashed pair
 # embedding, the experts of the size weighted at their input, their shared expert.
+# ``--design lumevik``: the Lumevik design beside Ravenex (the closest existing design: latent attention, several experts a
+# token with a choice bias).  Lumevik: layers in the order latent attention, attention, latent attention, attention
+# (heads of 128 with values of 128, a latent of 512, a query latent of 1,536; grouped-query attention with keys of 128 and
+# values of 64, a kv head for every four, a bias by distance up to 1,024, a window of 4,096 with four kept tokens, blended
+# values), the experts of the size in groups of four of which three are open, the shared expert behind a gate, the third
+# layer dense.  Ravenex at the same width, heads, latent, experts and dense layer, latent attention in every layer, a cache
+# of its own each, no token rows.
 DESIGN_SIZES = {
     "2k": dict(width=2048, heads=16, experts=16, top=4, expert_ff=1024, shared_ff=2048, dense_ff=8192),
     "5k": dict(width=5120, heads=40, experts=16, top=2, expert_ff=4096, shared_ff=8192, dense_ff=16384),
@@ -303,7 +310,30 @@ def nolapel_configs(sz, layers, window, vocab):
     return {"nolapel": nolapel, "tebalorn": tebalorn_configs(sz, layers, window, vocab)["tebalorn"]}
 
 
+def lumevik_configs(sz, layers, window, vocab):
+    H = sz["heads"]
+    latent = ("latent_attention", {"heads": H, "dim": 128, "vdim": 128, "kv_rank": 512, "q_rank": 1536, "scale": 128 ** -0.5})
+    attn = ("attention", {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 64, "scale": 128 ** -0.5, "bias_max": 1024,
+                          "mask": {"size": window, "keep_first": 4}, "v_mix": True})
+    router = {"experts": sz["experts"], "top": sz["top"]}
+    moe = {"kind": "moe", "router": dict(router, groups={"count": max(1, sz["experts"] // 4), "keep": max(1, sz["experts"] // 4 - 1)}),
+           "expert": {"ff": sz["expert_ff"], "limit": 7.0}, "shared": {"ff": sz["shared_ff"], "limit": 7.0}}
+    dense = {"kind": "dense", "ff": sz["dense_ff"], "limit": 7.0}
+    lumevik = {"architecture": "Lumevik", "vocab": vocab, "width": sz["width"], "norm": {"eps": 1e-6}, "torch_dtype": "bfloat16",
+               "layers": [dict(zip(("type", "mixer"), (latent, attn)[i % 2]), mlp=dense if i % 4 == 2 else moe) for i in range(layers)]}
+    mix = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "mask": {"size": window},
+           "rot": {"base": 10000.0, "dims": 64}, "scale": 192 ** -0.5}
+    r_moe = {"kind": "moe", "router": router, "expert": {"ff": sz["expert_ff"]}, "shared": {"ff": sz["shared_ff"]}}
+    ravenex = {"architecture": "Ravenex", "vocab": vocab, "width": sz["width"], "residual_mult": 0.7, "norm": {"eps": 1e-6},
+               "torch_dtype": "bfloat16",
+               "layers": [{"type": "latent_attention", "mixer": mix, "mlp": {"kind": "dense", "ff": sz["dense_ff"]} if i % 4 == 2 else r_moe}
+                          for i in range(layers)]}
+    return {"lumevik": lumevik, "ravenex": ravenex}
+
+
 def design_configs(sz, layers, window, vocab, design="ravenex"):
+    if design == "lumevik":
+        return lumevik_configs(sz, layers, window, vocab)
     if design == "nolapel":
         return nolapel_configs(sz, layers, window, vocab)
     if design == "pefedra":
@@ -338,7 +368,7 @@ def design_comparison(args):
     page, V, layers, window = 64, 32768, args.layers or 4, 4096
     batch, context, T = args.batch, args.context, args.prefill_tokens
     rng = np.random.RandomState(0)
-    beside = "Tebalorn" if args.design == "nolapel" else "Llama 4"
+    beside = {"nolapel": "Tebalorn", "lumevik": "Ravenex"}.get(args.design, "Llama 4")
     out = {"metric": f"prefill and decode tok/s of the {args.design.capitalize()} design beside {beside} at equal sizes (random weights)",
            "value": None, "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "dtype": args.dtype,
            "higher_is_better": True, "data": "synthetic: random weights, uniform-random token ids, context pages filled with random values",
@@ -667,9 +697,9 @@ def main() -> int:
     ap.add_argument("--workload", default="decode", choices=["decode", "longctx", "serve", "designs"],
                     help="designs: another design (--design) beside Llama 4 at equal sizes (see DESIGN_SIZES)")
     ap.add_argument("--design-sizes", default="2k,5k", help="designs: which of DESIGN_SIZES, comma separated")
-    ap.add_argument("--design", default="ravenex", choices=["ravenex", "pefedra", "tebalorn", "nolapel"],
+    ap.add_argument("--design", default="ravenex", choices=["ravenex", "pefedra", "tebalorn", "nolapel", "lumevik"],
                     help="designs: which design runs beside Llama 4 (pefedra: against Llama 4 with dense layers only; "
-                         "nolapel: beside Tebalorn, the closest existing design)")
+                         "nolapel: beside Tebalorn, lumevik: beside Ravenex, their closest existing designs)")
     ap.add_argument("--layers", type=int, default=None, help="fewer layers than the model has (memory or time)")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--context", type=int, default=4096)

@@ -24,9 +24,12 @@
 //   * runs that no column of the wave reads: skipped.
 // Optional per-head slopes (a score bias slope * (key - query position)) and a smooth cap on
 // the scores take the per-element path in an instantiation of their own.  A bias by distance from a
-// table (one number for every distance from the table's end on) has a third: runs within the table's
-// reach take the per-element path, with the tables of the kv head's query heads in LDS where they fit;
-// runs beyond it are whole runs whose scores all get the column's last table entry, in the exponent's fma.
+// table (one number for every distance from the table's end on) has a third: runs beyond the table's reach
+// are whole runs whose scores all get the column's last table entry, in the exponent's fma; whole runs within it
+// read the tables of the kv head's query heads from LDS, where they lie from the far end to the near (so that
+// consecutive keys read consecutive entries at fixed offsets from one address a run) with a margin at both ends
+// (so that the one address is all that has to be kept in bounds).  Tables too long for LDS take the
+// per-element path and are read from memory.
 //
 // Kept keys.  With a chunk or a window the first `keep` keys of the request may stay in sight: their
 // steps come before the rule's own, as edge steps.
@@ -55,6 +58,8 @@
 #define PF_COLS 256        // columns (query, head) per workgroup
 #define PF_KEYS 128        // keys per step
 #define PF_RUNS (PF_KEYS / 32)
+#define PF_TAB_FAR 32      // entries of a distance table in LDS beyond its last distance, all equal to that one's
+#define PF_TAB_NEAR 64     // entries below distance 0 (keys behind the query, which the mask takes out)
 
 enum { PF_PLAIN = 0, PF_EXTRA = 1, PF_DIST = 2 };
 // MODE: PF_EXTRA, score slopes or a cap are in use (every run takes the per-element path); PF_DIST, a
@@ -113,11 +118,15 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     const float slope = (EXTRA && slopes && live) ? slopes[head] * inv_scale : 0.f;
     // a bias by distance: this column's table (in LDS, or where it lies in memory) and its last entry, in the exponent's units
     const float* tab = DIST ? dist_bias + (size_t)(live ? head : 0) * n_dist : nullptr;
-    const int tab_at = DIST ? (live ? col % QH : 0) * tab_ld : 0;
     const int reach = DIST ? n_dist - 1 : 0;         // every key at least this far away gets the last entry
+    const int tab_at = DIST ? (live ? col % QH : 0) * tab_ld + reach + PF_TAB_FAR : 0;      // entry of distance 0 in LDS
     const float far_l2e = DIST ? tab[reach] * 1.4426950408889634f : 0.f;
-    if (DIST && tab_ld > 0)
-        for (int i = tid; i < QH * n_dist; i += 512) tab_sh[(i / n_dist) * tab_ld + i % n_dist] = dist_bias[(size_t)g * QH * n_dist + i];
+    if (DIST && tab_ld > 0) {
+        const int len = reach + PF_TAB_FAR + PF_TAB_NEAR;
+        for (int h = 0; h < QH; ++h)
+            for (int i = tid; i < len; i += 512)
+                tab_sh[h * tab_ld + i] = dist_bias[((size_t)g * QH + h) * n_dist + min(max(reach + PF_TAB_FAR - i, 0), reach)] * 1.4426950408889634f;
+    }
     bf16x8 qf[NS];
     {
         const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -147,19 +156,13 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
 #pragma unroll
         for (int i = 0; i < 16; ++i) o[d][i] = 0.f;
 
-    auto page_of = [&](int key) { const int i = key / ps; return i < max_blocks ? bt[i] : -1; };
+    auto page_of = [&](int key) __attribute__((always_inline)) { const int i = key / ps; return i < max_blocks ? bt[i] : -1; };
 
     // ---- staging: every wave sends its share of the step's tiles from the pages into LDS.  A
     // step has PF_RUNS runs of keys and as many of values, each HD/16 or VD/16 tiles of one kilobyte that
     // lie in a row in its page; a wave sends one run's keys or values, a tile a load (16 bytes a lane).
     static_assert(PF_RUNS == 4, "eight waves send four runs of keys and four of values");
     const int hx = wave >> 1, is_v = wave & 1;
-    auto send = [&](const bf16* src, bf16* dst, auto tiles) __attribute__((always_inline)) {
-#pragma unroll
-        for (int i = 0; i < decltype(tiles)::value; ++i)
-            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + i * 512 + lane * 8),
-                                             (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
-    };
     auto stage = [&](int u, int buf) __attribute__((always_inline)) {
         const int key = u * PF_KEYS + hx * 32;
         int pg = page_of(key);
@@ -167,9 +170,21 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         // values taken as zero
         pg = pg < 0 ? 0 : pg;
         // (value heads may be fewer than key heads: key head g reads value head g % Gv)
-        const int blk = (key % ps) >> 5;
-        if (is_v) send(v_pages + ((size_t)pg * Gv + g % Gv) * (size_t)ps * VD + (size_t)blk * VRUN, Vs + buf * VSTEP + hx * VRUN, std::integral_constant<int, VD / 16>{});
-        else send(k_pages + ((size_t)pg * G + g) * (size_t)ps * HD + (size_t)blk * RUN, Ks + buf * STEP + hx * RUN, std::integral_constant<int, HD / 16>{});
+        const int w = is_v ? VD : HD;
+        const bf16* src = (is_v ? v_pages + ((size_t)pg * Gv + g % Gv) * (size_t)ps * VD : k_pages + ((size_t)pg * G + g) * (size_t)ps * HD)
+            + (size_t)((key % ps) >> 5) * (32 * w) + lane * 8;
+        bf16* dst = (is_v ? Vs + buf * VSTEP : Ks + buf * STEP) + hx * (32 * w);
+        constexpr int LESS = HD < VD ? HD / 16 : VD / 16, MORE = HD < VD ? VD / 16 : HD / 16;
+#pragma unroll
+        for (int i = 0; i < LESS; ++i)
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + i * 512),
+                                             (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
+        if (MORE > LESS && w / 16 == MORE) {
+#pragma unroll
+            for (int i = LESS; i < MORE; ++i)
+                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + i * 512),
+                                                 (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
+        }
     };
 
     // this lane's part of the operand addresses: row r of tile tt, the lane's half of the k run
@@ -178,9 +193,13 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     const int v_lane = tt * 512 + hh * 128 + r * 8;
 
     // ---- one run (32 keys, from key0) out of LDS, run h of buffer `buf`.
-    // MASKED: tests per element.
-    auto run32 = [&](int key0, int buf, int h, auto masked_tag) __attribute__((always_inline)) {
-        constexpr bool MASKED = decltype(masked_tag)::value;
+    // RUN_WHOLE: every column reads all of it (with a distance table: beyond its reach); RUN_MASKED: tests per
+    // element; RUN_NEAR: every column reads all of it, the scores take the distance tables in LDS.
+    enum { RUN_WHOLE = 0, RUN_MASKED = 1, RUN_NEAR = 2 };
+    const int pq_at = live ? pq : pq_min;            // (a column without a query must not leave the tables either)
+    auto run32 = [&](int key0, int buf, int h, auto kind_tag) __attribute__((always_inline)) {
+        constexpr int KIND = decltype(kind_tag)::value;
+        constexpr bool MASKED = KIND == RUN_MASKED, TABLE = DIST && KIND != RUN_WHOLE;
         const bf16* kb_ = Ks + buf * STEP + h * RUN + k_lane;
         const bf16* vb_ = Vs + buf * VSTEP + h * VRUN + v_lane;
         f32x16 s;
@@ -210,6 +229,23 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                 for (int kg = 0; kg < 2; ++kg) vf[d][kg] = *(const bf16x8*)(vb_ + (2 * d) * 512 + kg * 256);
             __builtin_amdgcn_sched_group_barrier(0x100, 2 * NDT, 0);
         }
+        if (TABLE) {
+            // the scores in the exponent's units, with their biases; s[4j+i] is the key key0 + 8hh + 16(j&1) + 4(j>>1) + i
+            const int d0 = pq_at - key0 - hh * 8;
+            if (KIND == RUN_NEAR || tab_ld > 0) {
+                const float* te = tab_sh + tab_at - min(d0, reach + PF_TAB_FAR);
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) s[4 * j + i] = fmaf(s[4 * j + i], scale_log2e, te[(j & 1) * 16 + (j >> 1) * 4 + i]);
+            } else {
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i)
+                        s[4 * j + i] = fmaf(s[4 * j + i], scale_log2e, tab[min(max(d0 - (j & 1) * 16 - (j >> 1) * 4 - i, 0), reach)] * 1.4426950408889634f);
+            }
+        }
         bool absent = false;
         if (MASKED) {
             absent = page_of(key0) < 0;
@@ -227,10 +263,6 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
                         // the raw score is replaced by the one that the scale turns into the capped score
                         if (cap_ratio > 0.f) v = tanhf(v * cap_ratio) / cap_ratio;
                     }
-                    if (DIST) {
-                        const int d = min(max(pq - key, 0), reach);
-                        v += (tab_ld > 0 ? tab_sh[tab_at + d] : tab[d]) * inv_scale;
-                    }
                     const bool ok = sp_visible(key, pq, lo, keep);
                     s[4 * j + i] = ok ? (absent ? NAN : v) : -INFINITY;
                 }
@@ -244,8 +276,8 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
             mx = fmaxf(__uint_as_float(sw[0]), __uint_as_float(sw[1]));
         }
         // (a run out of the distance table's reach: all of its scores get the last entry)
-        const float c0 = DIST && !MASKED ? far_l2e : 0.f;
-        const float m_new = fmaxf(m_run, DIST ? fmaf(mx, scale_log2e, c0) : mx * scale_log2e);
+        const float c0 = DIST && KIND == RUN_WHOLE ? far_l2e : 0.f;
+        const float m_new = fmaxf(m_run, TABLE ? mx : (DIST ? fmaf(mx, scale_log2e, c0) : mx * scale_log2e));
         // a column with nothing visible so far keeps m = -inf: its weights are zero, not NaN
         const float m_safe = (MASKED && m_new == -INFINITY) ? 0.f : m_new;
         const float alpha = __builtin_amdgcn_exp2f(m_run - m_safe);
@@ -256,7 +288,7 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         for (int j = 0; j < 4; ++j)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                const float e = __builtin_amdgcn_exp2f(fmaf(s[4 * j + i], scale_log2e, m_off));
+                const float e = __builtin_amdgcn_exp2f(TABLE ? s[4 * j + i] + m_off : fmaf(s[4 * j + i], scale_log2e, m_off));
                 sum += e;
                 pf[j & 1][(j >> 1) * 4 + i] = (bf16)e;
             }
@@ -303,8 +335,8 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
             const int key0 = u * PF_KEYS + h * 32;
             if (key0 > pq_max || (key0 + 31 < lo_min && key0 >= keep)) continue;            // nothing here for this wave
             const bool whole = !EXTRA && (key0 >= lo_max || key0 + 31 < keep) && key0 + 31 <= pq_min - reach && page_of(key0) >= 0;
-            if (whole) run32(key0, buf, h, std::false_type{});
-            else run32(key0, buf, h, std::true_type{});
+            if (whole) run32(key0, buf, h, std::integral_constant<int, RUN_WHOLE>{});
+            else run32(key0, buf, h, std::integral_constant<int, RUN_MASKED>{});
         }
     };
 
@@ -317,14 +349,19 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
     // either into common registers in every run).  The kept keys' steps come before all others.  A split
     // takes its share of that order.
     const int n_keep = min((keep + PF_KEYS - 1) / PF_KEYS, u_first);
-    int uA = u_last + 1, uB = u_last + 1;
+    // (With distance tables the whole steps are those beyond their reach, uA .. uF-1, and, with the tables in
+    // LDS, those within it, uF .. uB-1, in a loop of their own again.)
+    int uA = u_last + 1, uB = u_last + 1, uF = u_last + 1;
     if (!EXTRA) {
         uA = max(u_first, (sp_first_visible(p_last, vis, span) + PF_KEYS - 1) / PF_KEYS);
-        uB = min(u_last + 1, max(p_first + 1 - reach, 0) / PF_KEYS);
+        uB = min(u_last + 1, (p_first + 1) / PF_KEYS);
+        uF = DIST ? min(uB, max(p_first + 1 - reach, 0) / PF_KEYS) : uB;
+        if (DIST && tab_ld == 0) uB = uF;
         if (uA >= uB) uA = uB = u_last + 1;
+        uF = max(uF, uA);
     }
     const int n_steps = n_keep + u_last + 1 - u_first, n_low = n_keep + uA - u_first, n_edge = n_steps - (uB - uA);
-    auto step_at = [&](int i) {
+    auto step_at = [u_first, n_keep, n_low, n_edge, uA, uB](int i) __attribute__((always_inline)) {
         return i < n_keep ? i : (i < n_low ? u_first + (i - n_keep) : (i < n_edge ? uB + (i - n_low) : uA + (i - n_edge)));
     };
     const int i_begin = (int)((long)n_steps * split / n_splits), i_end = (int)((long)n_steps * (split + 1) / n_splits);
@@ -350,16 +387,28 @@ void attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_
         for (int pg = k_lo / ps + lane; pg <= (k_hi - 1) / ps; pg += 64) bad |= pg >= max_blocks || bt[pg] < 0;
         poison = __any(bad);
     }
-    for (; i < i_end; ++i, buf ^= 1) {
+    const int i_near = DIST ? min(i_end, n_edge + (uF - uA)) : i_end;
+    for (; i < i_near; ++i, buf ^= 1) {
         const int u = uA + (i - n_edge);
         if (i + 1 < i_end) stage(u + 1, buf ^ 1);
         if (pq_max >= 0) {
 #pragma unroll
-            for (int h = 0; h < PF_RUNS; ++h) run32(u * PF_KEYS + h * 32, buf, h, std::false_type{});
+            for (int h = 0; h < PF_RUNS; ++h) run32(u * PF_KEYS + h * 32, buf, h, std::integral_constant<int, RUN_WHOLE>{});
         }
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
     }
+    if (DIST)
+        for (; i < i_end; ++i, buf ^= 1) {
+            const int u = uA + (i - n_edge);
+            if (i + 1 < i_end) stage(u + 1, buf ^ 1);
+            if (pq_max >= 0) {
+#pragma unroll
+                for (int h = 0; h < PF_RUNS; ++h) run32(u * PF_KEYS + h * 32, buf, h, std::integral_constant<int, RUN_NEAR>{});
+            }
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+            __syncthreads();
+        }
 
     // the two lanes of a column add their parts of the sum
     {
@@ -470,7 +519,7 @@ static int launch_prefill(const void* q, const void* k_pages, const void* v_page
     if (MODE == PF_DIST) {
         // a table row a head of the kv head, rows a part of the banks apart so that the heads of a wave's columns do not meet
         const int qh = H / G, apart = qh <= 32 ? 32 / qh : 1;
-        const long ld = ((long)n_dist + 31) / 32 * 32 + apart;
+        const long ld = ((long)n_dist + PF_TAB_FAR + PF_TAB_NEAR + 31) / 32 * 32 + apart;
         if (ld * qh * (long)sizeof(float) <= PF_TAB_BYTES) { tab_ld = (int)ld; sh += (size_t)ld * qh * sizeof(float); }
     }
     static bool allowed = false;          // one flag per instantiation: more LDS than the default limit

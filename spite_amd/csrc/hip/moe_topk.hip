@@ -19,6 +19,8 @@
 
 #define TOPK_MAX_PER_LANE 8      // up to 512 experts
 
+// NU: experts a lane, so that 64 * NU >= E.
+template <int NU>
 __global__ __launch_bounds__(256)
 void router_topk_kernel(const float* __restrict__ logits, const float* __restrict__ bias, int* __restrict__ expert,
                         float* __restrict__ weight, int T, int E, int ld, int top, int renorm, int mode,
@@ -26,9 +28,9 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
     const int lane = threadIdx.x & 63;
     const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
     if (t >= T) return;
-    float s[TOPK_MAX_PER_LANE], c[TOPK_MAX_PER_LANE];
+    float s[NU], c[NU];
 #pragma unroll
-    for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) {
+    for (int u = 0; u < NU; ++u) {
         const int e = lane + u * 64;
         s[u] = 0.f; c[u] = -INFINITY;
         if (e < E) {
@@ -39,16 +41,16 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
     if (mode == 2) {
         float zm = -INFINITY, zs = 0.f;
 #pragma unroll
-        for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) if (lane + u * 64 < E) zm = fmaxf(zm, s[u]);
+        for (int u = 0; u < NU; ++u) if (lane + u * 64 < E) zm = fmaxf(zm, s[u]);
         zm = wave_max(zm);
 #pragma unroll
-        for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) if (lane + u * 64 < E) { s[u] = expf(s[u] - zm); zs += s[u]; }
+        for (int u = 0; u < NU; ++u) if (lane + u * 64 < E) { s[u] = expf(s[u] - zm); zs += s[u]; }
         zs = 1.0f / wave_sum(zs);
 #pragma unroll
-        for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) s[u] *= zs;
+        for (int u = 0; u < NU; ++u) s[u] *= zs;
     }
 #pragma unroll
-    for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) {
+    for (int u = 0; u < NU; ++u) {
         const int e = lane + u * 64;
         if (e < E) {
             c[u] = s[u] + (bias ? bias[e] : 0.f);
@@ -58,11 +60,14 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
     if (n_groups > 1) {
         // the best group left is the group of the best expert of the groups left
         const int gs = E / n_groups;
+        int grp[NU];
+#pragma unroll
+        for (int u = 0; u < NU; ++u) grp[u] = (lane + u * 64) / gs;
         unsigned open = 0;                                  // bit u: this lane's expert u is in a group that stays
         for (int j = 0; j < keep_groups; ++j) {
             float best = -INFINITY; int be = 0x7fffffff;
 #pragma unroll
-            for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) {
+            for (int u = 0; u < NU; ++u) {
                 const int e = lane + u * 64;
                 if (e < E && !(open >> u & 1) && (c[u] > best || (c[u] == best && e < be))) { best = c[u]; be = e; }
             }
@@ -73,17 +78,17 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
             }
             const int gb = be / gs;
 #pragma unroll
-            for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) if (lane + u * 64 < E && (lane + u * 64) / gs == gb) open |= 1u << u;
+            for (int u = 0; u < NU; ++u) if (lane + u * 64 < E && grp[u] == gb) open |= 1u << u;
         }
 #pragma unroll
-        for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) if (!(open >> u & 1)) c[u] = -INFINITY;
+        for (int u = 0; u < NU; ++u) if (!(open >> u & 1)) c[u] = -INFINITY;
     }
     float sum = 0.f, top_z = -INFINITY;          // mode 1: the sum of exp(z - top_z) over the taken so far
     float mine_w = 0.f; int mine_e = 0;
     for (int j = 0; j < top; ++j) {
         float best = -INFINITY; int be = 0x7fffffff; float bs = 0.f;
 #pragma unroll
-        for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) {
+        for (int u = 0; u < NU; ++u) {
             const int e = lane + u * 64;
             if (e < E && (c[u] > best || (c[u] == best && e < be))) { best = c[u]; be = e; bs = s[u]; }
         }
@@ -94,7 +99,7 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
         }
         // a taken expert leaves the contest: its mark lies below every score
 #pragma unroll
-        for (int u = 0; u < TOPK_MAX_PER_LANE; ++u) if (lane + u * 64 == be) c[u] = -INFINITY;
+        for (int u = 0; u < NU; ++u) if (lane + u * 64 == be) c[u] = -INFINITY;
         if (mode == 1) {
             const float nz = fmaxf(top_z, bs);
             sum = sum * expf(top_z - nz) + expf(bs - nz);        // (exp(-inf) = 0 at the first)
@@ -126,7 +131,12 @@ extern "C" int spite_router_topk(const float* logits, const float* bias, int* ex
     SP_REQUIRE(T >= 0 && E > 0 && E <= 64 * TOPK_MAX_PER_LANE, "router_topk: %d experts, at most %d", E, 64 * TOPK_MAX_PER_LANE);
     SP_REQUIRE(top > 0 && top <= E, "router_topk: %d of %d experts", top, E);
     if (T == 0) return 0;
-    router_topk_kernel<<<(T + 3) / 4, 256, 0, st>>>(logits, bias, expert, weight, T, E, ld, top, renorm, mode, n_groups, keep_groups);
+#define SP_RT(NU) router_topk_kernel<NU><<<(T + 3) / 4, 256, 0, st>>>(logits, bias, expert, weight, T, E, ld, top, renorm, mode, n_groups, keep_groups)
+    if (E <= 64) SP_RT(1);
+    else if (E <= 128) SP_RT(2);
+    else if (E <= 256) SP_RT(4);
+    else SP_RT(TOPK_MAX_PER_LANE);
+#undef SP_RT
     SP_LAUNCH_CHECK("router_topk");
     return 0;
 }
