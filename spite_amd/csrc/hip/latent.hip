@@ -36,7 +36,7 @@ void latent_prepare_kernel(const T* __restrict__ qd, int ldq, const T* __restric
                            int H, int n, int r, int R, int rot_dims, int own,
                            int* __restrict__ rows_th, int* __restrict__ offsets_h, int T_all,
                            const T* __restrict__ cq_raw, int ld_cq, const float* __restrict__ w_cq, T* __restrict__ cq_out, int Q) {
-    __shared__ float red[4];
+    __shared__ float red[8];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int Dk = R + r, hw = n + r;
     const float pos = (float)positions[t];
@@ -53,18 +53,22 @@ void latent_prepare_kernel(const T* __restrict__ qd, int ldq, const T* __restric
         const int h = i / r, e = i - h * r;
         qa[((size_t)t * H + h) * Dk + R + e] = from_f32<T>(turned(row + (size_t)h * hw + n, e));
     }
+    // both norms' sums in one pass and one exchange
+    const T* cq = cq_raw + (size_t)t * ld_cq;
+    const T* dkv = dkv_all + (size_t)t * ld_dkv;
+    float sq_c = 0.f, sq = 0.f;
+    if (cq_out) for (int e = tid; e < Q; e += 256) { const float x = to_f32<T>(cq[e]); sq_c += x * x; }
+    if (own) for (int e = tid; e < R; e += 256) { const float x = to_f32<T>(dkv[e]); sq += x * x; }
+    sq_c = wave_sum(sq_c);
+    sq = wave_sum(sq);
+    if ((tid & 63) == 0) { red[tid >> 6] = sq_c; red[4 + (tid >> 6)] = sq; }
+    __syncthreads();
     if (cq_out) {
-        const T* cq = cq_raw + (size_t)t * ld_cq;
-        float sq = 0.f;
-        for (int e = tid; e < Q; e += 256) { const float x = to_f32<T>(cq[e]); sq += x * x; }
-        const float scale = 1.0f / sqrtf(block_sum<256>(sq, red) / (float)Q + eps);
+        const float scale = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)Q + eps);
         for (int e = tid; e < Q; e += 256) cq_out[(size_t)t * Q + e] = from_f32<T>(to_f32<T>(cq[e]) * scale * w_cq[e]);
     }
     if (own) {
-        const T* dkv = dkv_all + (size_t)t * ld_dkv;
-        float sq = 0.f;
-        for (int e = tid; e < R; e += 256) { const float x = to_f32<T>(dkv[e]); sq += x * x; }
-        const float scale = 1.0f / sqrtf(block_sum<256>(sq, red) / (float)R + eps);
+        const float scale = 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)R + eps);
         const int slot = slot_map[t];
         if (slot >= 0) {
             T* out = kv_pages + (size_t)slot * Dk;
