@@ -149,6 +149,7 @@ class LatentAttention(Mixer):
         prepare = lambda qd, own, query_latent: hipops.latent_prepare(
             qd, dkv if own else None, qa, cache.k_pages, ctx.positions, cache.slot_map, self.inv_freq, self.w_norm,
             self.eps, H, n, r, R, self.rot_dims, own, rows_th, offsets_h, query_latent=query_latent)
+        # (queries behind a latent are formed after this call; where it must name them, what it turns is turned again below)
         prepare(None if Q and self.own else q, self.own, latent)
         if Q:
             linear(latent[2], self.wq, q, ws=ws)
