@@ -22,13 +22,15 @@
 // whole q or k part again).  The row holds [HQ*D | GK*D | GV*Vd | ...] (`ld` elements to the next
 // row).  x = row + bias; with `wq` / `wk` the q and the k region are each divided by the root mean
 // square of the whole region and multiplied by their weights; then the first `rot` elements
-// of every q and k head turn by pos * inv_freq[i] in pairs (i, i + rot/2), sine and cosine both
+// of every q and k head turn by pos * inv_freq[i] in pairs (i, i + rot/2), or with `adjacent` (2i, 2i + 1), sine and cosine both
 // times `rot_mag` (1: a pure rotation; frequency scalings that stretch the context bring a
 // constant above 1 that sharpens the scores of the turning part); with `inv_freq_v` the
 // values turn by pos * inv_freq_v[m] in pairs (m, m + Vd/2).  Keys go to [page][GK][offset][Dp],
 // values to [page][GV][Vd][offset] (or the operand order of common.h).  Dp >= D is the width that
 // queries and keys are stored with: the elements behind D are written as zeros (a head narrower than
-// what an attention kernel takes is widened this way; zeros add nothing to a score).  With `v_other` (rows
+// what an attention kernel takes is widened this way; zeros add nothing to a score).  `head_norm`: every head is normed on
+// its own, with one weight vector for all heads or (`wq`, `wk` null) without weights.  A turn does not change a head's
+// root mean square, so without weights a norm before the rotation is the norm after it.  With `v_other` (rows
 // `ld_other` apart) the values are blended with another layer's of the same token before they are cached:
 // (1 - v_lam) v + v_lam other.
 template <typename T>
@@ -39,7 +41,7 @@ void qkv_prepare_kernel(const T* __restrict__ qkv, int ld, const float* __restri
                         const int* __restrict__ positions, const int* __restrict__ slot_map,
                         const float* __restrict__ inv_freq, int rot, float rot_mag, const float* __restrict__ inv_freq_v,
                         int HQ, int GK, int GV, int D, int Vd, int ps, int k_tiled, int v_tiled, int Dp, int hpb,
-                        int head_norm, float qt_coef, int qt_every, int v_from_k,
+                        int head_norm, int adjacent, float qt_coef, int qt_every, int v_from_k,
                         const T* __restrict__ v_other, int ld_other, float v_lam) {
     extern __shared__ float sm[];
     __shared__ float red[WIDE_NT / 64];
@@ -101,6 +103,7 @@ void qkv_prepare_kernel(const T* __restrict__ qkv, int ld, const float* __restri
         auto load = [&](int c) {
             float x = to_f32<T>(row[base + c]) + (bias ? bias[base + c] : 0.f);
             if (wn) x = x * sc * wn[wbase + c];
+            else if (head_norm) x *= sc;
             return x * qt;
         };
         T* dst = nullptr;
@@ -111,9 +114,10 @@ void qkv_prepare_kernel(const T* __restrict__ qkv, int ld, const float* __restri
             else dst[sp_k_index(off, c, Dp, k_tiled)] = from_f32<T>(v);
         };
         if (i < rh) {
-            const float a = load(i), b = load(i + rh);
-            store(i, a * cs[i] - b * sn[i]);
-            store(i + rh, b * cs[i] + a * sn[i]);
+            const int c1 = adjacent ? 2 * i : i, c2 = adjacent ? c1 + 1 : i + rh;
+            const float a = load(c1), b = load(c2);
+            store(c1, a * cs[i] - b * sn[i]);
+            store(c2, b * cs[i] + a * sn[i]);
         } else {
             const int c = rot + (i - rh);
             store(c, load(c));
@@ -156,7 +160,7 @@ void qkv_prepare_vec_kernel(const bf16* __restrict__ qkv, int ld, const float* _
                             const int* __restrict__ positions, const int* __restrict__ slot_map,
                             const float* __restrict__ inv_freq, int rot, float rot_mag, const float* __restrict__ inv_freq_v,
                             int HQ, int GK, int GV, int D, int Vd, int ps, int k_tiled, int v_tiled, int Dp, int hpb,
-                            int head_norm, float qt_coef, int qt_every, int v_from_k,
+                            int head_norm, int adjacent, float qt_coef, int qt_every, int v_from_k,
                             const bf16* __restrict__ v_other, int ld_other, float v_lam) {
     extern __shared__ __attribute__((aligned(16))) float sm[];
     __shared__ float red[WIDE_NT / 64];
@@ -205,7 +209,7 @@ void qkv_prepare_vec_kernel(const bf16* __restrict__ qkv, int ld, const float* _
     const size_t page = slot >= 0 ? (size_t)(slot / ps) : 0;
     const int off = slot >= 0 ? slot % ps : 0;
     // a head in groups of four: pairs that turn, elements that pass through, zeros behind D
-    const int pq = rh >> 2, sq = (D - rot) >> 2, zq = (Dp - D) >> 2, QI = pq + sq + zq;
+    const int pq = adjacent ? rot >> 2 : rh >> 2, sq = (D - rot) >> 2, zq = (Dp - D) >> 2, QI = pq + sq + zq;
     const int n_qk = (qk_hi > h_lo ? qk_hi - h_lo : 0) * QI;
     for (int it = tid; it < n_qk; it += WIDE_NT) {
         const int hh = h_lo + it / QI, j = it % QI;
@@ -218,6 +222,7 @@ void qkv_prepare_vec_kernel(const bf16* __restrict__ qkv, int ld, const float* _
         auto load = [&](int c) {
             f32x4 x = row4(base + c);
             if (wn) { const f32x4 ww = *(const f32x4*)(wn + wbase + c); x = x * sc * ww; }
+            else if (head_norm) x *= sc;
             return x * qt;
         };
         bf16* dst = is_q ? q_out + ((size_t)t * HQ + hh) * Dp : k_pages + (page * GK + (hh - HQ)) * (size_t)ps * Dp;
@@ -225,7 +230,12 @@ void qkv_prepare_vec_kernel(const bf16* __restrict__ qkv, int ld, const float* _
             const bf16x4 o = {(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
             *(bf16x4*)(dst + (is_q ? (size_t)c : sp_k_index(off, c, Dp, k_tiled))) = o;
         };
-        if (j < pq) {
+        if (j < pq && adjacent) {
+            const int c = j * 4, i = j * 2;                // two pairs
+            const f32x4 x = load(c);
+            store(c, f32x4{x[0] * cs[i] - x[1] * sn[i], x[1] * cs[i] + x[0] * sn[i],
+                           x[2] * cs[i + 1] - x[3] * sn[i + 1], x[3] * cs[i + 1] + x[2] * sn[i + 1]});
+        } else if (j < pq) {
             const int i = j * 4;
             const f32x4 a = load(i), b = load(i + rh);
             const f32x4 c4 = *(const f32x4*)(cs + i), s4 = *(const f32x4*)(sn + i);
@@ -263,7 +273,7 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
                                  float eps, void* q_out, void* k_pages, void* v_pages, const int* positions,
                                  const int* slot_map, const float* inv_freq, int rot, float rot_mag, const float* inv_freq_v,
                                  int T, int HQ, int GK, int GV, int D, int Vd, int page_size, int k_tiled, int v_tiled,
-                                 int Dp, int head_norm, float qt_coef, int qt_every, int v_from_k,
+                                 int Dp, int head_norm, int adjacent, float qt_coef, int qt_every, int v_from_k,
                                  const void* v_other, int ld_other, float v_lam, hipStream_t st) {
     if (Dp <= 0) Dp = D;
     SP_REQUIRE(Dp >= D, "qkv_prepare: heads of %d stored with %d elements", D, Dp);
@@ -271,7 +281,8 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
     SP_REQUIRE(ld >= (HQ + GK) * D + (v_from_k ? 0 : GV * Vd), "qkv_prepare: rows of %d elements for %d", ld, (HQ + GK) * D + (v_from_k ? 0 : GV * Vd));
     SP_REQUIRE(!v_from_k || (GV == GK && Vd == D && !inv_freq_v), "qkv_prepare: values taken from the keys have the keys' heads and width");
     SP_REQUIRE(!v_other || ld_other >= GV * Vd, "qkv_prepare: rows of %d values to blend with, %d wanted", ld_other, GV * Vd);
-    SP_REQUIRE(!head_norm || (wq && wk), "qkv_prepare: a head norm needs its two weight vectors");
+    SP_REQUIRE(!head_norm || (wq != nullptr) == (wk != nullptr), "qkv_prepare: a head norm has two weight vectors or none");
+    SP_REQUIRE(!head_norm || wq || rot_mag == 1.0f, "qkv_prepare: a head norm without weights goes with a pure rotation");
     SP_REQUIRE(qt_every >= 0, "qkv_prepare: query temperature every %d positions", qt_every);
     SP_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= D, "qkv_prepare: %d turning elements of a head of %d", rot, D);
     SP_REQUIRE(rot == 0 || inv_freq, "qkv_prepare: rotation needs a frequency table");
@@ -279,7 +290,7 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
     SP_REQUIRE(!slot_map || (k_pages && v_pages), "qkv_prepare: writing the cache needs its pages");
     SP_REQUIRE(!k_tiled || (dtype == SP_BF16 && Dp % 32 == 0 && page_size % 32 == 0), "qkv_prepare: keys of %d in operand order", Dp);
     SP_REQUIRE(!v_tiled || (dtype == SP_BF16 && Vd % 32 == 0 && page_size % 32 == 0), "qkv_prepare: values of %d in operand order", Vd);
-    SP_REQUIRE(eps > 0.f || (!wq && !wk), "qkv_prepare: the norm needs an eps");
+    SP_REQUIRE(eps > 0.f || (!wq && !wk && !head_norm), "qkv_prepare: the norm needs an eps");
     if (T == 0) return 0;
     const size_t sh = (size_t)(rot + (inv_freq_v ? Vd : 0)) * sizeof(float);
     SP_REQUIRE(sh <= 48 * 1024, "qkv_prepare: heads too wide");
@@ -291,22 +302,22 @@ extern "C" int spite_qkv_prepare(const void* qkv, int ld, int dtype, const float
     if (hpb > heads) hpb = heads;
     const dim3 grid(T, (unsigned)((heads + hpb - 1) / hpb));
     auto al = [](const void* p, int a) { return ((uintptr_t)p & (a - 1)) == 0; };
-    if (dtype == SP_BF16 && D % 4 == 0 && Dp % 4 == 0 && rot % 8 == 0 && ld % 4 == 0 && al(qkv, 8) && al(q_out, 8) && al(k_pages, 8)
+    if (dtype == SP_BF16 && D % 4 == 0 && Dp % 4 == 0 && rot % (adjacent ? 4 : 8) == 0 && ld % 4 == 0 && al(qkv, 8) && al(q_out, 8) && al(k_pages, 8)
         && al(bias, 16) && al(wq, 16) && al(wk, 16)) {
         // (the sine and cosine tables are read four at a time: the second starts rot/2 floats behind the first)
         qkv_prepare_vec_kernel<<<grid, WIDE_NT, sh, st>>>((const bf16*)qkv, ld, bias, wq, wk, eps, (bf16*)q_out, (bf16*)k_pages,
-            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k,
+            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, adjacent, qt_coef, qt_every, v_from_k,
             (const bf16*)v_other, ld_other, v_lam);
         SP_LAUNCH_CHECK("qkv_prepare");
         return 0;
     }
     if (dtype == SP_F32)
         qkv_prepare_kernel<float><<<grid, WIDE_NT, sh, st>>>((const float*)qkv, ld, bias, wq, wk, eps, (float*)q_out, (float*)k_pages,
-            (float*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k,
+            (float*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, adjacent, qt_coef, qt_every, v_from_k,
             (const float*)v_other, ld_other, v_lam);
     else if (dtype == SP_BF16)
         qkv_prepare_kernel<bf16><<<grid, WIDE_NT, sh, st>>>((const bf16*)qkv, ld, bias, wq, wk, eps, (bf16*)q_out, (bf16*)k_pages,
-            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, qt_coef, qt_every, v_from_k,
+            (bf16*)v_pages, positions, slot_map, inv_freq, rot, rot_mag, inv_freq_v, HQ, GK, GV, D, Vd, page_size, k_tiled, v_tiled, Dp, (int)hpb, head_norm, adjacent, qt_coef, qt_every, v_from_k,
             (const bf16*)v_other, ld_other, v_lam);
     else return sp_fail("qkv_prepare: unknown dtype %d", dtype);
     SP_LAUNCH_CHECK("qkv_prepare");

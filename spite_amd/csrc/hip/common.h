@@ -112,6 +112,17 @@ __device__ __forceinline__ float rows4_sum(float v) {
     return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
+// The sum over the 16 lanes of a row, by rotations within the row (no LDS traffic); every lane gets it.
+__device__ __forceinline__ float row16_sum(float x) {
+#define SP_ROR(n) __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), 0x120 | (n), 0xf, 0xf, false))
+    x += SP_ROR(8);
+    x += SP_ROR(4);
+    x += SP_ROR(2);
+    x += SP_ROR(1);
+#undef SP_ROR
+    return x;
+}
+
 // Sum over a workgroup of NT threads (NT a multiple of 64, at most 1024); every thread
 // gets the result.  `red` is shared scratch of at least NT/64 floats; two barriers.
 template <int NT>

@@ -65,17 +65,6 @@ extern "C" int spite_channel_decay(float* z, const float* bias, int T, int width
 
 template <int RR> struct la_block { static constexpr int tokens = RR == 16 ? 8 : 16; };
 
-// The sum over the 16 lanes of a row, by rotations within the row (no LDS traffic); every lane gets it.
-__device__ __forceinline__ float row16_sum(float x) {
-#define LA_ROR(n) __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), 0x120 | (n), 0xf, 0xf, false))
-    x += LA_ROR(8);
-    x += LA_ROR(4);
-    x += LA_ROR(2);
-    x += LA_ROR(1);
-#undef LA_ROR
-    return x;
-}
-
 // The sum over 32 lanes (two rows of 16): the rows' sums, then the lower row's into the upper row (a row's last
 // lane to the next row, rows 1 and 3 only).  The upper 16 of the 32 lanes get it.
 __device__ __forceinline__ float row32_sum(float x) {

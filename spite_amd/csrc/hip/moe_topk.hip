@@ -1,11 +1,13 @@
 // Routers that pick several experts a token, and what surrounds their grouped products.
 //
 // router_topk: from the router's fp32 logits z [T, E] the `top` experts with the largest choice
-// values are taken (the lowest index wins among equals), and each gets a weight.  Three ways of scoring:
+// values are taken (the lowest index wins among equals), and each gets a weight.  Four ways of scoring:
 //   sigmoid (mode 0): scores s = sigmoid(z); the choice goes by s + bias (bias may be null); an expert's
 //     weight is its score s without the bias, divided by the sum of the taken scores if `renorm`;
 //   softmax over the taken (mode 1): the choice goes by z + bias; the weights are the softmax of the taken
 //     experts' logits z alone (they add up to one; `renorm` has nothing left to do);
+//   softmax over the taken, bias inside (mode 3): z + bias are the logits themselves: the choice goes by them and the
+//     weights are their softmax over the taken;
 //   softmax over all (mode 2): scores s = softmax(z) over every expert; choice and weights as with sigmoid.
 // With `n_groups` > 1 the experts form equal groups of neighbours and only those of the `keep_groups` groups whose
 // largest choice value is largest can be taken (the lowest group among equals).  The logits' rows may lie `ld` apart.
@@ -36,8 +38,10 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
         if (e < E) {
             const float z = logits[(size_t)t * ld + e];
             s[u] = mode == 0 ? 1.0f / (1.0f + expf(-z)) : z;
+            if (mode == 3 && bias) s[u] += bias[e];
         }
     }
+    if (mode == 3) { bias = nullptr; mode = 1; }
     if (mode == 2) {
         float zm = -INFINITY, zs = 0.f;
 #pragma unroll
@@ -123,7 +127,7 @@ void router_topk_kernel(const float* __restrict__ logits, const float* __restric
 
 extern "C" int spite_router_topk(const float* logits, const float* bias, int* expert, float* weight, int T, int E, int ld, int top,
                                  int renorm, int mode, int n_groups, int keep_groups, hipStream_t st) {
-    SP_REQUIRE(mode >= 0 && mode <= 2, "router_topk: scoring %d", mode);
+    SP_REQUIRE(mode >= 0 && mode <= 3, "router_topk: scoring %d", mode);
     SP_REQUIRE(ld >= E, "router_topk: rows of %d logits for %d experts", ld, E);
     SP_REQUIRE(n_groups >= 1 && E > 0 && E % n_groups == 0 && keep_groups >= 1 && keep_groups <= n_groups, "router_topk: %d of %d groups of %d experts",
                keep_groups, n_groups, E);

@@ -1,5 +1,5 @@
-// Small row-wise kernels: the token shift of a mixer's input, an activation applied in place and a
-// constant on fp32 rows (the logits of a model whose output has one).
+// Small row-wise kernels: the token shift of a mixer's input, an activation applied in place, a constant on fp32 rows
+// (the logits of a model whose output has one), and a sigmoid gate element by element.
 #include "common.h"
 
 // ------------------------------------------------------------------ token shift
@@ -115,5 +115,48 @@ extern "C" int spite_scale_rows(float* x, size_t n, float c, hipStream_t st) {
     const int blocks = (int)((n + 255) / 256 < 16384 ? (n + 255) / 256 : 16384);
     scale_rows_kernel<<<blocks, 256, 0, st>>>(x, n, c);
     SP_LAUNCH_CHECK("scale_rows");
+    return 0;
+}
+
+// ------------------------------------------------------------------ a gate, element by element
+// y[t][c] = x[t][c] * sigmoid(gate[t][c]) in fp32; x and y dense [T, n] (y may be x), gate rows `ldg` apart, all of one
+// type.
+template <typename T>
+__global__ __launch_bounds__(256)
+void gate_rows_kernel(const T* x, const T* __restrict__ gate, int ldg, T* y, size_t total, int n) {
+    const size_t stride = (size_t)gridDim.x * 256;
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < total; i += stride) {
+        const size_t t = i / n, c = i - t * n;
+        y[i] = from_f32<T>(to_f32<T>(x[i]) / (1.0f + expf(-to_f32<T>(gate[t * ldg + c]))));
+    }
+}
+
+// eight bfloat16 a thread
+__global__ __launch_bounds__(256)
+void gate_rows_bf16x8_kernel(const bf16* x, const bf16* __restrict__ gate, int ldg, bf16* y, size_t total8, int n8) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= total8) return;
+    const size_t t = i / n8, c = (i - t * n8) * 8;
+    const bf16x8 a = *(const bf16x8*)(x + i * 8), g = *(const bf16x8*)(gate + t * ldg + c);
+    bf16x8 o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) o[e] = (bf16)((float)a[e] / (1.0f + expf(-(float)g[e])));
+    *(bf16x8*)(y + i * 8) = o;
+}
+
+extern "C" int spite_gate_rows(const void* x, const void* gate, int ldg, void* y, int dtype, int T, int n, hipStream_t st) {
+    SP_REQUIRE(T >= 0 && n > 0 && ldg >= n, "gate_rows: rows of %d, gate rows %d apart", n, ldg);
+    const size_t total = (size_t)T * n;
+    if (total == 0) return 0;
+    auto al = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    if (dtype == SP_BF16 && n % 8 == 0 && ldg % 8 == 0 && al(x) && al(gate) && al(y) && (total / 8 + 255) / 256 < (1u << 31)) {
+        gate_rows_bf16x8_kernel<<<(unsigned)((total / 8 + 255) / 256), 256, 0, st>>>((const bf16*)x, (const bf16*)gate, ldg, (bf16*)y, total / 8, n / 8);
+    } else {
+        const int blocks = (int)((total + 255) / 256 < 16384 ? (total + 255) / 256 : 16384);
+        if (dtype == SP_F32) gate_rows_kernel<float><<<blocks, 256, 0, st>>>((const float*)x, (const float*)gate, ldg, (float*)y, total, n);
+        else if (dtype == SP_BF16) gate_rows_kernel<bf16><<<blocks, 256, 0, st>>>((const bf16*)x, (const bf16*)gate, ldg, (bf16*)y, total, n);
+        else return sp_fail("gate_rows: unknown dtype %d", dtype);
+    }
+    SP_LAUNCH_CHECK("gate_rows");
     return 0;
 }

@@ -77,12 +77,15 @@ def lib():
             "spite_router_topk": [P, P, P, P, I, I, I, I, I, I, I, I, P],
             "spite_moe_combine": [P, P, P, P, I, P, I, I, I, P],
             "spite_gated_rows": [P, I, P, P, I, I, I, P, I, I, P],
-            "spite_qkv_prepare": [P, I, I, P, P, P, F, P, P, P, P, P, P, I, F, P, I, I, I, I, I, I, I, I, I, I, I, F, I, I, P, I, F, P],
+            "spite_qkv_prepare": [P, I, I, P, P, P, F, P, P, P, P, P, P, I, F, P, I, I, I, I, I, I, I, I, I, I, I, I, F, I, I, P, I, F, P],
             "spite_attn_wide": [P, P, P, P, I, I, P, P, P, I, I, I, I, I, I, I, I, I, I, F, I, I, P, P, I, P, I, P],
             "spite_attn_finish": [P, I, P, I, P, P, P, I, I, I, I, I, F, F, F, P],
             "spite_token_shift": [P, P, I, P, P, P, P, P, I, I, I, P],
             "spite_act_rows": [P, I, c_size_t, I, P],
             "spite_scale_rows": [P, c_size_t, F, P],
+            "spite_gate_rows": [P, P, I, P, I, I, I, P],
+            "spite_delta_gates": [P, P, I, I, P, I, P, I, I, P, P, F, F, P, P, I, I, I, I, P],
+            "spite_delta_scan": [P, P, P, I, I, I, I, P, P, P, I, P, P, I, P, I, I, I, I, I, P],
             "spite_channel_decay": [P, P, I, I, F, I, P],
             "spite_linear_attn_scan": [P, P, P, I, I, I, I, P, P, F, P, I, P, P, I, P, I, I, I, I, I, I, P, P, P],
             "spite_gated_group_norm": [P, P, I, P, I, P, I, I, I, I, F, I, I, P, I, P, I, P],
@@ -694,16 +697,17 @@ def latent_prepare(qd, dkv, qa, kv_pages, positions, slot_map, inv_freq, w_norm,
     the per-head products.  ``qd`` None: the queries come later (their latent is normed here first) or have no
     rotated part; qa is left alone.  ``query_latent`` = (raw [T, >= Q] rows, weight fp32 [Q], out [T, Q]): out = the raw
     rows RMS-normed (the same eps) times the weight."""
-    if qd is None and (dkv is None or not own):
-        raise KernelError("latent_prepare: neither queries nor cache rows to prepare")
-    T = (dkv if qd is None else qd).shape[0]
+    lead = qd if qd is not None else dkv if dkv is not None and own else query_latent[0] if query_latent is not None else None
+    if lead is None:
+        raise KernelError("latent_prepare: neither queries nor a query latent nor cache rows to prepare")
+    T = lead.shape[0]
     Dk = R + r
     Q, raw, w_q, out_q = 0, None, None, None
     if query_latent is not None:
         raw, w_q, out_q = query_latent
         Q = w_q.numel()
         if raw.dim() != 2 or raw.stride(1) != 1 or raw.shape[0] < T or raw.shape[1] < Q or tuple(out_q.shape) != (T, Q) \
-                or raw.dtype != out_q.dtype or raw.dtype != (dkv if qd is None else qd).dtype:
+                or raw.dtype != out_q.dtype or raw.dtype != lead.dtype:
             raise KernelError(f"latent_prepare: query latent {tuple(raw.shape)} to {tuple(out_q.shape)} with a weight of {Q}")
     if qd is None:
         pass
@@ -715,7 +719,7 @@ def latent_prepare(qd, dkv, qa, kv_pages, positions, slot_map, inv_freq, w_norm,
         raise KernelError("latent_prepare: outputs or positions too small")
     if rot_dims and inv_freq.numel() < rot_dims // 2:
         raise KernelError("latent_prepare: frequency table shorter than the turning pairs")
-    dt = (dkv if qd is None else qd).dtype
+    dt = lead.dtype
     if own:
         if kv_pages.dim() != 4 or kv_pages.shape[1] != 1 or kv_pages.shape[3] != Dk or slot_map.numel() < T or w_norm.numel() != R:
             raise KernelError(f"latent_prepare: pages {tuple(kv_pages.shape)} for rows of {Dk}, or slots / norm weight too small")
@@ -752,7 +756,7 @@ def attn_latent_generic(q, kv_pages, out, positions, seq_of_token, block_table, 
 
 
 # -------------------------------------------------------------------------------------------- several experts a token
-ROUTER_SCORING = {"sigmoid": 0, "softmax_taken": 1, "softmax": 2}
+ROUTER_SCORING = {"sigmoid": 0, "softmax_taken": 1, "softmax": 2, "softmax_taken_biased": 3}
 
 
 def router_topk(logits, bias, expert, weight, top, renorm=False, scoring="sigmoid", groups=None, n_experts=None):
@@ -760,7 +764,7 @@ def router_topk(logits, bias, expert, weight, top, renorm=False, scoring="sigmoi
     score + bias (bias fp32 [E] or None; lowest index among equals) into expert[T*top], their
     scores (without the bias; divided by their sum with ``renorm``) into weight[T*top].  With
     ``scoring`` = ``softmax_taken`` the choice goes by z + bias and the weights are the softmax over the
-    taken experts' logits; ``softmax``: scores softmax(z) over all experts, the rest as with sigmoid.  ``groups`` =
+    taken experts' logits (``softmax_taken_biased``: over the taken experts' z + bias, the bias being part of the logits); ``softmax``: scores softmax(z) over all experts, the rest as with sigmoid.  ``groups`` =
     (count, keep): only experts of the ``keep`` groups (``count`` equal groups of neighbours) whose largest choice
     value is largest can be taken.  ``n_experts``: the logits are the first so many columns of the rows."""
     T, E = logits.shape[0], int(n_experts or logits.shape[1])
@@ -862,7 +866,7 @@ def attn_latent_mfma(q, kv_pages, out, positions, seq_of_token, block_table, wg,
 def qkv_prepare(qkv, q_out, k_pages, v_pages, positions, slot_map, HQ, GK, GV, D, Vd, page_size, *, bias=None,
                 norm_q=None, norm_k=None, eps=0.0, inv_freq=None, rot=0, inv_freq_v=None, write_kv=True,
                 k_tiled=False, v_tiled=False, stored_dim=None, rot_magnitude=1.0, head_norm=False, q_temperature=None,
-                values_from_keys=False, blend=None):
+                values_from_keys=False, blend=None, adjacent=False):
     """Between a fused projection and the cache (see attn_wide.hip).  qkv: rows that begin with
     [HQ*D | GK*D | GV*Vd] (further columns are left alone); ``bias`` fp32 over those; ``norm_q`` /
     ``norm_k`` (fp32 [HQ*D], [GK*D]): weights of an RMS norm over the whole q and the whole k part;
@@ -871,7 +875,8 @@ def qkv_prepare(qkv, q_out, k_pages, v_pages, positions, slot_map, HQ, GK, GV, D
     pairs (m, m + Vd/2).  q_out
     [T, HQ*Dp]; key pages [pages, GK, page_size, Dp]; value pages [pages, GV, Vd, page_size], with
     Dp = ``stored_dim`` (default D): queries and keys are stored that wide, zeros behind their D.
-    ``head_norm``: ``norm_q`` / ``norm_k`` hold D weights each and every head is normed on its own.
+    ``head_norm``: ``norm_q`` / ``norm_k`` hold D weights each, or are None (no weights), and every head is normed on its
+    own.  ``adjacent``: the pairs that turn are (2i, 2i + 1).
     ``q_temperature`` = (coef, every): the queries (after their norm) times 1 + coef * ln(floor((p + 1) / every) + 1)
     at position p.  ``values_from_keys``: the row holds no values, [HQ*D | GK*D] only; the values are the keys as
     the row holds them, before norm and rotation (GV = GK, Vd = D).  ``blend`` = (other [T, >= GV*Vd] in the rows'
@@ -912,7 +917,7 @@ def qkv_prepare(qkv, q_out, k_pages, v_pages, positions, slot_map, HQ, GK, GV, D
         _ptr(positions, "positions", torch.int32), _ptr(slot_map, "slot_map", torch.int32) if write_kv else None,
         _ptr(inv_freq, "inv_freq", torch.float32, True), int(rot), float(rot_magnitude),
         _ptr(inv_freq_v, "inv_freq_v", torch.float32, True),
-        T, HQ, GK, GV, D, Vd, page_size, int(bool(k_tiled)), int(bool(v_tiled)), Dp, int(bool(head_norm)), qt_coef, qt_every,
+        T, HQ, GK, GV, D, Vd, page_size, int(bool(k_tiled)), int(bool(v_tiled)), Dp, int(bool(head_norm)), int(bool(adjacent)), qt_coef, qt_every,
         int(bool(values_from_keys)), other.data_ptr() if other is not None else None, other.stride(0) if other is not None else 0,
         float(lam), _stream()), "qkv_prepare")
 
@@ -993,6 +998,16 @@ def act_rows(x, act):
 def scale_rows(x, c: float):
     """x *= c in place; x fp32."""
     _check(lib().spite_scale_rows(_ptr(x, "x", torch.float32), x.numel(), float(c), _stream()), "scale_rows")
+
+
+def gate_rows(x, gate, y):
+    """y = x * sigmoid(gate) element by element, in fp32; x and y dense [T, n] of one dtype (y may be x), gate a
+    [T, >= n] view of it whose rows may lie apart."""
+    T, n = x.shape
+    if y.shape != x.shape or y.dtype != x.dtype or gate.dtype != x.dtype:
+        raise KernelError(f"gate_rows: x {tuple(x.shape)} {x.dtype}, gate {gate.dtype}, y {tuple(y.shape)} {y.dtype}")
+    pg, ldg = _rows_view(gate, "gate", n, T)
+    _check(lib().spite_gate_rows(_ptr(x, "x"), pg, ldg, _ptr(y, "y"), dtype_code(x.dtype), T, n, _stream()), "gate_rows")
 
 
 # -------------------------------------------------------------------------------------------- linear attention
@@ -1240,3 +1255,46 @@ def bias_rows(y, v, out):
         raise KernelError("bias_rows: shapes")
     f = torch.float32
     _check(lib().spite_bias_rows(_ptr(y, "y", f), _ptr(v, "v", f), _ptr(out, "out", f), T, d, _stream()), "bias_rows")
+
+
+# -------------------------------------------------------------------------------------------- gated delta rule
+def delta_gates(q, k, raw_a, raw_b, a_log, dt_bias, qk_scale, gates, G, H, D, q_scale=1.0, eps=1e-6):
+    """The fp32 numbers beside the rows of the delta rule (see delta_rule.hip): qk_scale [T, 2, G]: q_scale /
+    sqrt(sum q^2 + eps) and 1 / sqrt(sum k^2 + eps) of every q/k head; gates [T, 2, H]: log g = -exp(a_log) *
+    softplus(raw_a + dt_bias), and beta = sigmoid(raw_b).  q, k [T, G*D] and raw_a, raw_b [T, H]: views of one dtype whose
+    rows may lie apart."""
+    f = torch.float32
+    if tuple(qk_scale.shape[1:]) != (2, G) or tuple(gates.shape[1:]) != (2, H) or gates.shape[0] != qk_scale.shape[0]:
+        raise KernelError(f"delta_gates: qk_scale {tuple(qk_scale.shape)}, gates {tuple(gates.shape)} for G={G} H={H}")
+    T = gates.shape[0]
+    if len({q.dtype, k.dtype, raw_a.dtype, raw_b.dtype}) != 1 or a_log.numel() != H or dt_bias.numel() != H:
+        raise KernelError("delta_gates: rows of one dtype, one a_log and dt_bias a head")
+    (pq, ldq), (pk, ldk) = _rows_view(q, "q", G * D, T), _rows_view(k, "k", G * D, T)
+    (pa, lda), (pb, ldb) = _rows_view(raw_a, "raw_a", H, T), _rows_view(raw_b, "raw_b", H, T)
+    _check(lib().spite_delta_gates(pq, pk, ldq, ldk, pa, lda, pb, ldb, dtype_code(q.dtype), _ptr(a_log, "a_log", f), _ptr(dt_bias, "dt_bias", f),
+                                   float(q_scale), float(eps), _ptr(qk_scale, "qk_scale", f), _ptr(gates, "gates", f), T, G, H, D, _stream()),
+           "delta_gates")
+
+
+def _delta_checks(q, k, v, qk_scale, gates, state, out, G, H, D, V, what):
+    T = gates.shape[0]
+    if q.dtype != k.dtype or q.dtype != v.dtype or H % G:
+        raise KernelError(f"{what}: q, k and v of one dtype, {H} heads over {G} of q and k")
+    if tuple(qk_scale.shape) != (T, 2, G) or tuple(gates.shape) != (T, 2, H) or tuple(state.shape[1:]) != (H, D, V) or out.numel() < T * H * V:
+        raise KernelError(f"{what}: qk_scale {tuple(qk_scale.shape)}, gates {tuple(gates.shape)}, state {tuple(state.shape)} for G={G} H={H} D={D} V={V}")
+    return _rows_view(q, "q", G * D, T), _rows_view(k, "k", G * D, T), _rows_view(v, "v", H * V, T)
+
+
+def delta_scan(q, k, v, qk_scale, gates, state, out, cu_seqlens, seq_slots, n_seqs, G, H, D, V, single=False):
+    """The gated delta rule over every entry of the step, token by token: S <- g S; u = beta (v - S^T k); S <- S + k u^T;
+    o = S^T q, with q and k times their factors.  q, k [T, G*D], v [T, H*V] (views, rows may lie apart); ``qk_scale``,
+    ``gates`` as ``delta_gates`` leaves them; state fp32 [slots, H, D, V], read and written at the entries' slots; out fp32
+    [T, H*V].  ``single``: every entry holds one token (a kernel of its own)."""
+    (pq, ldq), (pk, ldk), (pv, ldv) = _delta_checks(q, k, v, qk_scale, gates, state, out, G, H, D, V, "delta_scan")
+    f = torch.float32
+    if cu_seqlens.numel() < n_seqs + 1 or seq_slots.numel() < n_seqs or (single and gates.shape[0] != n_seqs):
+        raise KernelError("delta_scan: metadata too small, or more tokens than entries in a step of single tokens")
+    _check(lib().spite_delta_scan(pq, pk, pv, ldq, ldk, ldv, dtype_code(q.dtype), _ptr(qk_scale, "qk_scale", f), _ptr(gates, "gates", f),
+                                  _ptr(state, "state", f), state.shape[0], _ptr(cu_seqlens, "cu_seqlens", torch.int32),
+                                  _ptr(seq_slots, "seq_slots", torch.int32), int(n_seqs), _ptr(out, "out", f), H, G, D, V,
+                                  int(bool(single)), _stream()), "delta_scan")

@@ -188,7 +188,7 @@ class ParallelBlock(Block):
     ``spec.extra["shift"]`` (a PartSpec of category ``shift``, optional) stands between the first norm
     and the mixer and keeps a state row per request; the feed-forward may be missing;
     ``spec.extra["side"]`` (category ``side``, optional) adds its input from the step's tokens to the
-    stream after both.  The results are handed to the next block, whose first norm adds them."""
+    stream after both.  A mixer with several caches (``Mixer.cache_needs``) gets them by name.  The results are handed to the next block, whose first norm adds them."""
     graph_safe = True
 
     def __init__(self, env, spec):
@@ -215,7 +215,8 @@ class ParallelBlock(Block):
         self.step_arrays = tuple(sorted({a for _, part, _ in self.children for a in part.step_arrays}))
 
     def cache_needs(self):
-        needs = {"mixer": self.mixer.cache_need()}
+        # a mixer with one cache: under "mixer"; one with several (``Mixer.cache_needs``): under its own names
+        needs = {name or "mixer": need for name, need in self.mixer.cache_needs().items()}
         if self.shift is not None and self.shift.state_need() is not None:
             from .base import CacheNeed
             needs["shift"] = CacheNeed(state=self.shift.state_need())
@@ -288,7 +289,10 @@ class ParallelBlock(Block):
         state["ffn_in"] = (n, n32 if self.ffn.wants_f32_input and logits is None else None, logits)
 
     def _stage_mixer(self, state, ctx, cache):
-        state["mixed"] = run_mixer(self.mixer, state.pop("mixer_in"), state, ctx, cache["mixer"] if isinstance(cache, dict) else cache)
+        mine = cache
+        if isinstance(cache, dict) and "mixer" in cache:
+            mine = cache["mixer"]
+        state["mixed"] = run_mixer(self.mixer, state.pop("mixer_in"), state, ctx, mine)
 
     def _stage_ffn(self, state, ctx, cache):
         pend = (state.pop("mixed"),)

@@ -32,7 +32,8 @@ with a bound of their own each (``activation="clamped"``, ``limit``, ``shared_li
 min(g, L) sigmoid(1.702 min(g, L)) (clamp(u, -L, L) + 1).
 
 ``moe_topk_softmax``: the same part with the other way of scoring: the ``top_k`` experts with the largest
-logits are taken and their weights are the softmax over the taken logits alone; no bias.
+logits are taken and their weights are the softmax over the taken logits alone; with ``logit_bias`` a bias per expert is
+part of the logits.
 """
 from __future__ import annotations
 
@@ -237,7 +238,7 @@ class MoeTopKSigmoid(FeedForward):
                  shared_gate=False, limit=None, shared_limit=None):
         """``scoring``: ``sigmoid`` (the choice by sigmoid(z) + bias, weights sigmoid(z)), ``softmax`` (the same with the
         softmax over all experts) or ``softmax_taken`` (the choice by z + bias, weights the softmax over the taken
-        experts' z).  ``groups``: (count, keep); ``shared_gate``, ``limit``, ``shared_limit``: see above.  ``weight_input``: the weight multiplies
+        experts' z) or ``softmax_taken_biased`` (the bias is part of the logits: choice and softmax by z + bias).  ``groups``: (count, keep); ``shared_gate``, ``limit``, ``shared_limit``: see above.  ``weight_input``: the weight multiplies
         the expert's input instead of its output: the result is the sum of expert(w * x)."""
         self.weight_input = bool(weight_input)
         if scoring not in hipops.ROUTER_SCORING:
@@ -321,7 +322,9 @@ class MoeTopKSigmoid(FeedForward):
             if self.scoring == "softmax" and not self.renormalize:
                 raise ValueError("moe: given experts under a softmax over all of them need renormalized weights")
             logits = torch.full_like(logits, float("-inf")).scatter_(1, take, logits.gather(1, take))
-            bias = groups = None
+            groups = None
+            if self.scoring != "softmax_taken_biased":
+                bias = None
         hipops.router_topk(logits, bias, expert, weight, k, renorm=self.renormalize, scoring=self.scoring, groups=groups,
                            n_experts=E)
         if trace is not None:                         # a testing aid: which experts each token took, [T, top_k]
@@ -350,9 +353,11 @@ class MoeTopKSigmoid(FeedForward):
 
 @register("ffn", "moe_topk_softmax")
 class MoeTopKSoftmax(MoeTopKSigmoid):
-    """Several experts a token, taken by their logits and weighted by the softmax over the taken ones."""
+    """Several experts a token, taken by their logits and weighted by the softmax over the taken ones.  ``logit_bias``:
+    a learned number an expert (``correction``) is part of its logit, in the choice and in the softmax."""
 
     def __init__(self, env, hidden_size, intermediate_size, n_experts, top_k, shared_intermediate_size=None,
-                 activation="silu"):
+                 activation="silu", logit_bias=False, limit=None, shared_limit=None):
         super().__init__(env, hidden_size, intermediate_size, n_experts, top_k, shared_intermediate_size,
-                         score_bias=False, renormalize=False, activation=activation, scoring="softmax_taken")
+                         score_bias=bool(logit_bias), renormalize=False, activation=activation,
+                         scoring="softmax_taken_biased" if logit_bias else "softmax_taken", limit=limit, shared_limit=shared_limit)

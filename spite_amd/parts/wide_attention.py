@@ -16,7 +16,8 @@ keys and queries ``key_dim`` wide, values ``value_dim`` wide, with, each as an o
   head's values, times ``1 - diff``; lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff is one number
   of the layer, formed from four vectors of the checkpoint when it is loaded;
 * ``head_gate``: head h's result times sigmoid(W_g x)_h (``gate_proj`` [H, d]), before the output
-  projection;
+  projection; ``head_gate="elements"``: every element of the heads' results times a sigmoid of its own (``gate_proj``
+  [H*value_dim, d]);
 * ``sinks``: every head's softmax has one more term in its denominator, exp(s_h) with a learned number
   s_h per head (``sink`` [H]): it is no key, is not scaled, brings no value and counts once, so a head
   may give less than all of its weight to the keys it sees; ``sinks="zero"``: the term is exp(0) = 1 for
@@ -24,8 +25,9 @@ keys and queries ``key_dim`` wide, values ``value_dim`` wide, with, each as an o
 * ``conv_taps`` >= 1: a short causal convolution over time on every channel of the q and of the k projection
   (``q_conv`` [H*key_dim, taps], ``k_conv`` [G*key_dim, taps], the last column the token's own), right after the
   projection; the last taps - 1 projected rows of a request are its state between steps;
-* ``head_norm``: an RMS norm of every q and k head on its own, with one weight vector for all heads
-  (``q_norm``, ``k_norm`` [key_dim]);
+* ``head_norm``: an RMS norm of every q and k head on its own before the rotation, with one weight vector for all heads
+  (``q_norm``, ``k_norm`` [key_dim]); ``head_norm="unit"``: without weights (before or after the rotation is then the same,
+  a turn leaves a head's root mean square as it is);
 * ``q_temperature`` = (coef, every): the normed queries at position p times 1 + coef ln(floor((p+1)/every) + 1);
 * ``values="keys"``: there is no value projection; the values are the keys as they leave the convolution,
   before their norm (``value_dim`` = ``key_dim``);
@@ -70,6 +72,10 @@ class WideAttention(Mixer):
             raise ValueError(f"wide_attention: {visibility} of size {span}")
         if maps not in (1, 2):
             raise ValueError(f"wide_attention: {maps} score maps a head")
+        if head_gate not in (False, True, None, "elements"):
+            raise ValueError(f"wide_attention: head_gate {head_gate!r} (known: True, 'elements')")
+        if head_norm not in (False, True, None, "unit"):
+            raise ValueError(f"wide_attention: head_norm {head_norm!r} (known: True, 'unit')")
         if maps == 2 and (value_position is not None or head_gate or sinks):
             raise ValueError("wide_attention: two score maps go with neither turned values nor a head gate nor sinks")
         if values not in ("projection", "keys"):
@@ -94,11 +100,13 @@ class WideAttention(Mixer):
         self.value_blend = value_blend
         self.blend = 0.0
         self.bias, self.projection_norm, self.head_gate = bool(bias), bool(projection_norm), bool(head_gate)
+        self.gate_elements = head_gate == "elements"
         self.sinks = bool(sinks)
         self.zero_sinks = sinks == "zero"
         self.w_sink = None
         self.taps = max(int(conv_taps or 0), 0)             # 1: a weight per channel on the token's own row, no state
         self.head_norm, self.values_from_keys = bool(head_norm), values == "keys"
+        self.norm_weights = self.projection_norm or head_norm is True
         self.q_temperature = None if not q_temperature else (float(q_temperature[0]), int(q_temperature[1]))
         if self.q_temperature is not None and self.q_temperature[1] < 1:
             raise ValueError(f"wide_attention: query temperature every {self.q_temperature[1]} positions")
@@ -107,8 +115,12 @@ class WideAttention(Mixer):
         self.position = build_part("position", position, env) if position is not None else None
         self.value_position = build_part("position", value_position, env) if value_position is not None else None
         for pe in (self.position, self.value_position):
-            if pe is not None and (not pe.fused or pe.kernel_args().get("adjacent")):
-                raise ValueError("wide_attention: the position encoding must be a rotation in halves")
+            if pe is not None and not pe.fused:
+                raise ValueError("wide_attention: the position encoding must be a rotation")
+        if self.value_position is not None and self.value_position.kernel_args().get("adjacent"):
+            raise ValueError("wide_attention: the values turn in halves")
+        if head_norm == "unit" and self.position is not None and self.position.kernel_args().get("magnitude", 1.0) != 1.0:
+            raise ValueError("wide_attention: a norm per head without weights goes with a pure rotation")
         self.HQ, self.GK = self.H * self.maps, self.G * self.maps
         # the MFMA kernels take certain pairs of key and value widths: narrower keys (and queries) are stored
         # as wide as the next one in a bfloat16 run, zeros behind their own elements
@@ -119,7 +131,7 @@ class WideAttention(Mixer):
         self.n_qkv = self.n_qk + (0 if self.values_from_keys else self.G * self.Vd)
         self.w_in = self.wo = self.b_in = self.w_qnorm = self.w_knorm = None
         self.inv_freq = self.inv_freq_v = None
-        self.rot = 0
+        self.rot, self.adjacent = 0, False
         self.rot_magnitude = 1.0
         self.lam = 0.0
 
@@ -132,7 +144,7 @@ class WideAttention(Mixer):
         if self.taps:
             p.update({"q_conv": ParamSpec((H * D, self.taps), kind="vector", init="normal"),
                       "k_conv": ParamSpec((G * D, self.taps), kind="vector", init="normal")})
-        if self.head_norm:
+        if self.head_norm and self.norm_weights:
             p.update({"q_norm": ParamSpec((D,), kind="vector", init="ones"), "k_norm": ParamSpec((D,), kind="vector", init="ones")})
         if self.bias:
             p.update({"q_bias": ParamSpec((H * m * D,), kind="vector", init="normal"),
@@ -144,7 +156,7 @@ class WideAttention(Mixer):
         if self.maps == 2:
             p.update({k: ParamSpec((D,), kind="vector", init="normal") for k in ("lambda_q1", "lambda_k1", "lambda_q2", "lambda_k2")})
         if self.head_gate:
-            p["gate_proj"] = ParamSpec((H, d))
+            p["gate_proj"] = ParamSpec((H * Vd if self.gate_elements else H, d))
         if self.score_position is not None:
             p.update(self.score_position.params())
         if self.value_blend is not None:
@@ -176,7 +188,7 @@ class WideAttention(Mixer):
         self.wo = Weight(t["o_proj"])
         if self.bias:
             self.b_in = torch.cat([self._by_map(t["q_bias"], H), self._by_map(t["k_bias"], G), t["v_bias"]]).float().contiguous()
-        if self.projection_norm or self.head_norm:
+        if self.norm_weights:
             self.w_qnorm, self.w_knorm = t["q_norm"].float().contiguous(), t["k_norm"].float().contiguous()
         if self.taps:
             # tap by tap, [taps, channels]: the kernel's loads of one tap are consecutive
@@ -197,7 +209,7 @@ class WideAttention(Mixer):
             ka = self.position.kernel_args()
             if ka["use_rope"]:
                 self.inv_freq, self.rot = ka["inv_freq"], int(ka.get("rotary_dim") or self.D)
-                self.rot_magnitude = float(ka.get("magnitude", 1.0))
+                self.rot_magnitude, self.adjacent = float(ka.get("magnitude", 1.0)), bool(ka.get("adjacent"))
                 if self.rot > self.D:
                     raise ValueError(f"wide_attention: {self.rot} turning elements in heads of {self.D}")
         if self.value_position is not None:
@@ -282,7 +294,8 @@ class WideAttention(Mixer):
                            cache.page_size, bias=self.b_in, norm_q=self.w_qnorm, norm_k=self.w_knorm, eps=self.eps,
                            inv_freq=self.inv_freq, rot=self.rot, inv_freq_v=self.inv_freq_v, write_kv=cache.write,
                            k_tiled=cache.tiled, v_tiled=cache.tiled, stored_dim=Dk, rot_magnitude=self.rot_magnitude,
-                           head_norm=self.head_norm, q_temperature=self.q_temperature, values_from_keys=self.values_from_keys, blend=blend)
+                           head_norm=self.head_norm, q_temperature=self.q_temperature, values_from_keys=self.values_from_keys, blend=blend,
+                           adjacent=self.adjacent)
         if cache.tiled and self._mfma(cache.page_size):
             a = ws.take((T, HQ * Vd), x.dtype)
             cu_tail, lead = ctx.derived[TAIL]
@@ -299,13 +312,16 @@ class WideAttention(Mixer):
                              T, HQ, GK, G, Dk, Vd, cache.page_size, self.visibility, self.span, self.scale,
                              k_tiled=cache.tiled, v_tiled=cache.tiled, sinks=self.w_sink, slopes=self.slopes, keep=self.keep,
                              dist_bias=self.dist_bias)
-        if self.maps == 2 or self.inv_freq_v is not None or self.head_gate:
+        each = self.gate_elements
+        if self.maps == 2 or self.inv_freq_v is not None or (self.head_gate and not each):
             o = ws.take((T, H * Vd), x.dtype)
-            gate = proj[:, self.n_qkv:self.n_qkv + H] if self.head_gate else None
+            gate = proj[:, self.n_qkv:self.n_qkv + H] if self.head_gate and not each else None
             hipops.attn_finish(a, o, ctx.positions, H, Vd, maps=self.maps, lam=self.lam, eps=self.eps,
                                post=1.0 - self.diff, inv_freq_v=self.inv_freq_v, gate=gate)
         else:
             o = a
+        if each:
+            hipops.gate_rows(o, proj[:, self.n_qkv:self.n_qkv + H * Vd], o)
         out = ws.take((T, self.d), torch.float32)
         linear(o, self.wo, out, ws=ws)
         return out
