@@ -254,3 +254,351 @@ extern "C" int spite_delta_scan(const void* q, const void* k, const void* v, int
     SP_LAUNCH_CHECK("delta_scan");
     return 0;
 }
+
+// ------------------------------------------------------------------ prompts, 32 tokens at a time, on the matrix units
+// Within a chunk let G_t be the sum of log g over its tokens up to t, and write k_t = sk_t K_t, q_t = sq_t Q_t with the
+// bfloat16 rows K, Q and their fp32 factors.  With the state S0 before the chunk,
+//
+//   u_t = beta_t (v_t - exp(G_t) S0^T k_t - sum_(s<t) exp(G_t - G_s) (k_t.k_s) u_s)
+//   o_t = exp(G_t) S0^T q_t + sum_(s<=t) exp(G_t - G_s) (q_t.k_s) u_s
+//   S   = exp(G_C) S0 + sum_s k_s (exp(G_C - G_s) u_s)^T
+//
+// so U = (I + A)^-1 R with the strictly lower triangular A_ts = beta_t exp(G_t - G_s) (k_t.k_s) and the rows
+// R_t = beta_t v_t - beta_t exp(G_t) S0^T k_t.  Every exponent is a sum of logarithms of decays, never above 0.
+//
+// The first kernel forms, for every chunk and head at once, what does not depend on the state: (I + A)^-1 (by substitution),
+// the matrix M of the second line and the factors of the rows; and K^T in operand order.  The second walks a head's chunks.
+//
+// Nothing is rounded to bfloat16 on the way: K and Q *are* bfloat16 (their factors are applied to the products' rows),
+// and an fp32 operand that meets them (the state, U) is split into three bfloat16 summands, 8 bits each, that add up to
+// its 24 bits, so the products on the bfloat16 units are those of the fp32 numbers, summed in fp32; the small products
+// whose both operands are fp32 (the inverse and M times 16 columns) run on the fp32 units.  Sums of logarithms are
+// fp64, so that a difference of two of them keeps its bits however far both are from 0.
+//
+// Layouts.  A wave holds 16 value columns; a state tile (j, tt) of 16 rows is the key channels 32 j + 8 a + 4 tt + r in the
+// register r of lane (a, column), so that the tiles' registers of a lane are the 8 consecutive channels that the lane
+// supplies as the right operand of the next product: the state never moves between lanes.  The same holds for U (a
+// lane's 4 + 4 tokens): its products take their tokens in the order in which the lanes hold them.
+#define DC_C 32                                      // tokens a chunk
+#define DC_TILE 256                                  // floats of a 16 x 16 tile
+#define DC_REC (6 * DC_TILE + 4 * DC_C + 8)          // a chunk's and head's record: inverse and M, three tiles each
+                                                     // (0,0) (1,0) (1,1), the rows' factors, exp(G_C)
+typedef unsigned dc_u4 __attribute__((ext_vector_type(4)));
+
+// element (t, s) of a 16 x 16 tile in the order of the fp32 products' left operand: lane (s/4, t), register s%4
+__device__ __forceinline__ int dc_pos(int t, int s) { return (((s >> 2) * 16 + t) << 2) + (s & 3); }
+
+// 64 threads a (chunk, head).
+template <int KD>
+__global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(3)))
+void delta_chunk_prepare_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k, int ldq, int ldk, const float* __restrict__ qk_scale,
+                                const float* __restrict__ gates, const int* __restrict__ chunk_t0, const int* __restrict__ chunk_n,
+                                bf16* __restrict__ kt, float* __restrict__ rec, int H, int G) {
+    constexpr int D = 32 * KD, LK = D + 8;
+    __shared__ __attribute__((aligned(16))) bf16 krow[DC_C * LK];
+    __shared__ __attribute__((aligned(16))) float at[DC_C][DC_C + 4];       // A transposed: at[s][t]
+    __shared__ float diag[2][16][17];
+    __shared__ double gsum[DC_C];
+    __shared__ float f_q[DC_C], f_k[DC_C], f_b[DC_C];
+    const int c = blockIdx.x, h = blockIdx.y, lane = threadIdx.x, row = lane & 15, a = lane >> 4;
+    const int t0 = chunk_t0[c], n = chunk_n[c], g = h / (H / G);
+    // the tokens' factors; behind the chunk's last token: no decay, nothing written, nothing read
+    {
+        const int i = lane & 31;
+        const bool ok = i < n;
+        const size_t t = t0 + (ok ? i : 0);
+        double s = ok ? (double)gates[t * 2 * H + h] : 0.0;
+#pragma unroll
+        for (int o = 1; o < 32; o <<= 1) { const double up = __shfl_up(s, o, 32); if (i >= o) s += up; }
+        if (lane < 32) {
+            gsum[i] = s;
+            f_b[i] = ok ? gates[t * 2 * H + H + h] : 0.f;
+            f_q[i] = ok ? qk_scale[t * 2 * G + g] : 0.f;
+            f_k[i] = ok ? qk_scale[t * 2 * G + G + g] : 0.f;
+        }
+    }
+    bf16x8 ka[2][KD], qa[2][KD];
+#pragma unroll
+    for (int ti = 0; ti < 2; ++ti)
+#pragma unroll
+        for (int j = 0; j < KD; ++j) {
+            const int i = 16 * ti + row;
+            const bool ok = i < n;
+            const size_t t = t0 + (ok ? i : 0);
+            const int d = 32 * j + 8 * a;
+            const dc_u4 x = *(const dc_u4*)(k + t * ldk + (size_t)g * D + d), y = *(const dc_u4*)(q + t * ldq + (size_t)g * D + d);
+            ka[ti][j] = __builtin_bit_cast(bf16x8, ok ? x : dc_u4{0, 0, 0, 0});
+            qa[ti][j] = __builtin_bit_cast(bf16x8, ok ? y : dc_u4{0, 0, 0, 0});
+            *(bf16x8*)(krow + i * LK + d) = ka[ti][j];
+        }
+    f32x4 kk[3], qk[3];                               // tiles (0,0) (1,0) (1,1)
+#pragma unroll
+    for (int x = 0; x < 3; ++x) { kk[x] = f32x4{0.f, 0.f, 0.f, 0.f}; qk[x] = kk[x]; }
+#pragma unroll
+    for (int j = 0; j < KD; ++j)
+#pragma unroll
+        for (int x = 0; x < 3; ++x) {
+            const int ti = x > 0, tj = x > 1;
+            kk[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[ti][j], ka[tj][j], kk[x], 0, 0, 0);
+            qk[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qa[ti][j], ka[tj][j], qk[x], 0, 0, 0);
+        }
+    __syncthreads();
+    float* out = rec + ((size_t)c * H + h) * DC_REC;
+#pragma unroll
+    for (int x = 0; x < 3; ++x) {
+        const int ti = x > 0, tj = x > 1, s = 16 * tj + row;
+        f32x4 av;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int tl = 4 * a + r, t = 16 * ti + tl;
+            const float ratio = t >= s ? expf((float)(gsum[t] - gsum[s])) * f_k[s] : 0.f;
+            av[r] = t > s ? f_b[t] * f_k[t] * ratio * kk[x][r] : 0.f;
+            out[3 * DC_TILE + x * DC_TILE + dc_pos(tl, row)] = f_q[t] * ratio * qk[x][r];
+        }
+        *(f32x4*)&at[s][16 * ti + 4 * a] = av;
+    }
+    if (lane < 32) {
+        const float eg = expf((float)gsum[lane]);
+        float* fr = out + 6 * DC_TILE;
+        fr[lane] = f_b[lane];
+        fr[DC_C + lane] = f_b[lane] * eg * f_k[lane];
+        fr[2 * DC_C + lane] = eg * f_q[lane];
+        fr[3 * DC_C + lane] = expf((float)(gsum[DC_C - 1] - gsum[lane])) * f_k[lane];
+        if (lane == 0) fr[4 * DC_C] = expf((float)gsum[DC_C - 1]);
+    }
+    __syncthreads();
+    // the inverse of the two diagonal tiles by substitution, lane (tile, column): x_t = [t = column] - sum_(s<t) A_ts x_s
+    if (lane < 32) {
+        float x[16];
+#pragma unroll
+        for (int t = 0; t < 16; ++t) x[t] = t == row ? 1.f : 0.f;
+#pragma unroll
+        for (int s = 0; s < 15; ++s) {
+#pragma unroll
+            for (int t4 = (s + 1) / 4; t4 < 4; ++t4) {
+                const f32x4 w = *(const f32x4*)&at[16 * a + s][16 * a + t4 * 4];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) if (t4 * 4 + r > s) x[t4 * 4 + r] = fmaf(-w[r], x[s], x[t4 * 4 + r]);
+            }
+            asm volatile("" ::: "memory");           // (the reads of later columns stay where they are: registers)
+        }
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            out[2 * a * DC_TILE + dc_pos(t, row)] = x[t];
+            diag[a][t][row] = x[t];
+        }
+    }
+    __syncthreads();
+    // the tile below: - T11 (A10 T00)
+    {
+        f32x4 y = {0.f, 0.f, 0.f, 0.f}, z = y;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) y = __builtin_amdgcn_mfma_f32_16x16x4f32(at[4 * a + r][16 + row], diag[0][4 * a + r][row], y, 0, 0, 0);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) z = __builtin_amdgcn_mfma_f32_16x16x4f32(diag[1][row][4 * a + r], y[r], z, 0, 0, 0);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) out[DC_TILE + dc_pos(4 * a + r, row)] = -z[r];
+    }
+    if (h % (H / G) == 0) {
+        // K^T as the left operand of the state's update: lane (a, row) of tile (j, tt) holds channel 32 j + 8 (row/4) + 4 tt + row%4
+        // of the tokens 4 a .. 4 a + 3 and 16 + 4 a ..
+        bf16* dst = kt + ((size_t)c * G + g) * (2 * KD * 512);
+#pragma unroll
+        for (int x = 0; x < 2 * KD; ++x) {
+            const int d = 32 * (x >> 1) + 8 * (row >> 2) + 4 * (x & 1) + (row & 3);
+            bf16x8 o;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] = krow[((e & 4) * 4 + 4 * a + (e & 3)) * LK + d];
+            *(bf16x8*)(dst + (x * 64 + lane) * 8) = o;
+        }
+    }
+}
+
+// The three bfloat16 summands of eight fp32 numbers.
+__device__ __forceinline__ void dc_split(const f32x4& x, const f32x4& y, bf16x8& hi, bf16x8& mid, bf16x8& lo) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const float v = e < 4 ? x[e & 3] : y[e & 3];
+        hi[e] = (bf16)v;
+        const float r = v - (float)hi[e];
+        mid[e] = (bf16)r;
+        lo[e] = (bf16)(r - (float)mid[e]);
+    }
+}
+
+// 256 threads take 64 value columns of one head of one entry, a wave 16 of them, and walk the entry's chunks; the next
+// chunk's operands are on their way in registers while this one is computed from LDS.
+template <int KD>
+__global__ __launch_bounds__(256)
+void delta_chunk_scan_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k, const bf16* __restrict__ v, int ldq, int ldk, int ldv,
+                             const int* __restrict__ first_chunk, const int* __restrict__ chunk_t0, const int* __restrict__ chunk_n,
+                             const bf16* __restrict__ kt, const float* __restrict__ rec, float* __restrict__ state,
+                             const int* __restrict__ seq_slots, float* __restrict__ out, int H, int G, int V) {
+    constexpr int D = 32 * KD, NO = 128 * KD;             // 16-byte pieces of one operand (K, Q, K^T)
+    constexpr int PIECES = 3 * NO + DC_REC / 4, NP = (PIECES + 255) / 256;
+    static_assert(DC_REC % 4 == 0, "a record is whole pieces");
+    __shared__ __attribute__((aligned(16))) dc_u4 lds[PIECES];
+    const int e = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, a = lane >> 4;
+    const int g = h / (H / G), col = blockIdx.z * 64 + (tid >> 6) * 16 + (lane & 15);
+    const bool cok = col < V;
+    const bool busy = blockIdx.z * 64 + (tid >> 6) * 16 < V;        // the wave has a column at all
+    const int c_lo = first_chunk[e], c_hi = first_chunk[e + 1];
+    if (c_lo >= c_hi) return;
+    float* sbase = state + ((size_t)seq_slots[e] * H + h) * (size_t)D * V + col;
+    f32x4 S[2 * KD];
+#pragma unroll
+    for (int x = 0; x < 2 * KD; ++x)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[x][r] = cok ? sbase[(size_t)(32 * (x >> 1) + 8 * a + 4 * (x & 1) + r) * V] : 0.f;
+    dc_u4 st[NP];
+    float vn[2][4];
+    // operands of chunk c on their way: K and Q rows in the order of a product's left operand, K^T and the record as they lie
+#define DC_FETCH(c)                                                                                                     \
+    {                                                                                                                   \
+        const int t0 = chunk_t0[c], n = chunk_n[c];                                                                     \
+        _Pragma("unroll")                                                                                               \
+        for (int u = 0; u < NP; ++u) {                                                                                  \
+            const int p = tid + u * 256;                                                                                \
+            if (p < 2 * NO) {                                                                                           \
+                const int o = p % NO, i = 16 * (o / (64 * KD)) + (o & 15), d = 32 * ((o >> 6) % KD) + 8 * ((o >> 4) & 3); \
+                const bool ok = i < n;                                                                                  \
+                const size_t t = t0 + (ok ? i : 0);                                                                     \
+                const dc_u4 got = *(const dc_u4*)((p < NO ? k + t * ldk : q + t * ldq) + (size_t)g * D + d);             \
+                st[u] = ok ? got : dc_u4{0, 0, 0, 0};                                                                   \
+            } else if (p < 3 * NO) {                                                                                    \
+                st[u] = *((const dc_u4*)(kt + ((size_t)(c) * G + g) * (2 * KD * 512)) + (p - 2 * NO));                   \
+            } else if (p < PIECES) {                                                                                    \
+                st[u] = *((const dc_u4*)(rec + ((size_t)(c) * H + h) * DC_REC) + (p - 3 * NO));                          \
+            }                                                                                                           \
+        }                                                                                                               \
+        _Pragma("unroll")                                                                                               \
+        for (int x = 0; x < 8; ++x) {                                                                                   \
+            const int i = 16 * (x >> 2) + 4 * a + (x & 3);                                                              \
+            const bool ok = i < n && cok;                                                                               \
+            const bf16 got = v[(size_t)(t0 + (ok ? i : 0)) * ldv + (size_t)h * V + (ok ? col : 0)];                     \
+            vn[x >> 2][x & 3] = ok ? (float)got : 0.f;                                                                  \
+        }                                                                                                               \
+    }
+    DC_FETCH(c_lo)
+    const bf16x8* kop = (const bf16x8*)lds;
+    const bf16x8* qop = kop + NO;
+    const bf16x8* ktop = qop + NO;
+    const f32x4* inv = (const f32x4*)(lds + 3 * NO);
+    const f32x4* mm = inv + 3 * 64;
+    const f32x4* fr = mm + 3 * 64;                         // the rows' factors, four tokens each
+    for (int c = c_lo; c < c_hi; ++c) {
+        __syncthreads();                                   // the chunk before has been read
+#pragma unroll
+        for (int u = 0; u < NP; ++u) if (tid + u * 256 < PIECES) lds[tid + u * 256] = st[u];
+        f32x4 vv[2];
+#pragma unroll
+        for (int x = 0; x < 8; ++x) vv[x >> 2][x & 3] = vn[x >> 2][x & 3];
+        __syncthreads();
+        const int t0 = chunk_t0[c], n = chunk_n[c];
+        if (c + 1 < c_hi) DC_FETCH(c + 1)
+        if (!busy) continue;
+        // S0^T k and S0^T q, the smallest summands first
+        f32x4 R[2], O[2];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) { R[i] = f32x4{0.f, 0.f, 0.f, 0.f}; O[i] = R[i]; }
+#pragma unroll
+        for (int j = 0; j < KD; ++j) {
+            bf16x8 s3[3];
+            dc_split(S[2 * j], S[2 * j + 1], s3[2], s3[1], s3[0]);
+#pragma unroll
+            for (int y = 0; y < 3; ++y)
+#pragma unroll
+                for (int i = 0; i < 2; ++i) {
+                    R[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kop[(i * KD + j) * 64 + lane], s3[y], R[i], 0, 0, 0);
+                    O[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qop[(i * KD + j) * 64 + lane], s3[y], O[i], 0, 0, 0);
+                }
+        }
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+            const f32x4 b4 = fr[4 * i + a], c4 = fr[8 + 4 * i + a], e4 = fr[16 + 4 * i + a];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                R[i][r] = b4[r] * vv[i][r] - c4[r] * R[i][r];
+                O[i][r] *= e4[r];
+            }
+        }
+        // U = (I + A)^-1 R, then O += M U
+        f32x4 U[2];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) U[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int x = 0; x < 3; ++x) {
+            const int ti = x > 0, tj = x > 1;
+            const f32x4 w = inv[x * 64 + lane];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) U[ti] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[r], R[tj][r], U[ti], 0, 0, 0);
+        }
+#pragma unroll
+        for (int x = 0; x < 3; ++x) {
+            const int ti = x > 0, tj = x > 1;
+            const f32x4 w = mm[x * 64 + lane];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) O[ti] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[r], U[tj][r], O[ti], 0, 0, 0);
+        }
+        // S <- exp(G_C) S + K (factors U)^T
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+            const f32x4 f4 = fr[24 + 4 * i + a];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) U[i][r] *= f4[r];
+        }
+        bf16x8 u3[3];
+        dc_split(U[0], U[1], u3[2], u3[1], u3[0]);
+        const float whole = fr[32][0];
+#pragma unroll
+        for (int x = 0; x < 2 * KD; ++x) {
+            const bf16x8 w = ktop[x * 64 + lane];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) S[x][r] *= whole;
+#pragma unroll
+            for (int y = 0; y < 3; ++y) S[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, u3[y], S[x], 0, 0, 0);
+        }
+#pragma unroll
+        for (int x = 0; x < 8; ++x) {
+            const int i = 16 * (x >> 2) + 4 * a + (x & 3);
+            if (i < n && cok) out[(size_t)(t0 + i) * H * V + (size_t)h * V + col] = O[x >> 2][x & 3];
+        }
+    }
+#undef DC_FETCH
+    if (!cok) return;
+#pragma unroll
+    for (int x = 0; x < 2 * KD; ++x)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sbase[(size_t)(32 * (x >> 1) + 8 * a + 4 * (x & 1) + r) * V] = S[x][r];
+}
+
+// Bytes of scratch for n_chunks chunks: K^T in operand order, then the records.
+extern "C" size_t spite_delta_chunk_workspace(int n_chunks, int H, int G, int D) {
+    return (size_t)n_chunks * ((size_t)G * D * DC_C * sizeof(bf16) + (size_t)H * DC_REC * sizeof(float));
+}
+extern "C" int spite_delta_chunk_tokens() { return DC_C; }
+
+// chunks: int32 [n_seqs + 1] the first chunk of every entry, [n_chunks] the chunks' first tokens, [n_chunks] their lengths.
+extern "C" int spite_delta_chunk(const void* q, const void* k, const void* v, int ldq, int ldk, int ldv, const float* qk_scale, const float* gates,
+                                 float* state, int n_slots, const int* chunks, int n_chunks, const int* seq_slots, int n_seqs,
+                                 void* scratch, float* out, int H, int G, int D, int V, hipStream_t st) {
+    SP_REQUIRE(n_seqs >= 0 && n_chunks >= 0 && H > 0 && G > 0 && H % G == 0 && V > 0 && n_slots > 0, "delta_chunk: bad sizes H=%d G=%d V=%d", H, G, V);
+    SP_REQUIRE(D == 32 || D == 64 || D == 96 || D == 128, "delta_chunk: %d key channels a head (32, 64, 96 or 128)", D);
+    SP_REQUIRE(ldq >= G * D && ldk >= G * D && ldv >= H * V, "delta_chunk: rows shorter than the heads");
+    SP_REQUIRE(H <= 65535 && (V + 63) / 64 <= 65535, "delta_chunk: too many heads or value columns");
+    auto on16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    SP_REQUIRE(ldq % 8 == 0 && ldk % 8 == 0 && on16(q) && on16(k) && on16(scratch), "delta_chunk: q and k rows must start on 16 bytes");
+    if (n_seqs == 0 || n_chunks == 0) return 0;
+    bf16* kt = (bf16*)scratch;
+    float* rec = (float*)(kt + (size_t)n_chunks * G * D * DC_C);
+    const int *first = chunks, *t0 = chunks + n_seqs + 1, *n = t0 + n_chunks;
+#define DC_RUN(KD) do { \
+        delta_chunk_prepare_kernel<KD><<<dim3(n_chunks, H), 64, 0, st>>>((const bf16*)q, (const bf16*)k, ldq, ldk, qk_scale, gates, t0, n, kt, rec, H, G); \
+        SP_LAUNCH_CHECK("delta_chunk_prepare"); \
+        delta_chunk_scan_kernel<KD><<<dim3(n_seqs, H, (V + 63) / 64), 256, 0, st>>>((const bf16*)q, (const bf16*)k, (const bf16*)v, ldq, ldk, ldv, \
+            first, t0, n, kt, rec, state, seq_slots, out, H, G, V); } while (0)
+    if (D == 32) DC_RUN(1); else if (D == 64) DC_RUN(2); else if (D == 96) DC_RUN(3); else DC_RUN(4);
+#undef DC_RUN
+    SP_LAUNCH_CHECK("delta_chunk");
+    return 0;
+}

@@ -85,6 +85,8 @@ def lib():
             "spite_scale_rows": [P, c_size_t, F, P],
             "spite_gate_rows": [P, P, I, P, I, I, I, P],
             "spite_delta_gates": [P, P, I, I, P, I, P, I, I, P, P, F, F, P, P, I, I, I, I, P],
+            "spite_delta_chunk": [P, P, P, I, I, I, P, P, P, I, P, I, P, I, P, P, I, I, I, I, P],
+            "spite_delta_chunk_tokens": [],
             "spite_delta_scan": [P, P, P, I, I, I, I, P, P, P, I, P, P, I, P, I, I, I, I, I, P],
             "spite_channel_decay": [P, P, I, I, F, I, P],
             "spite_linear_attn_scan": [P, P, P, I, I, I, I, P, P, F, P, I, P, P, I, P, I, I, I, I, I, I, P, P, P],
@@ -107,6 +109,8 @@ def lib():
             fn.restype = c_int
         l.spite_attn_prefill_workspace.argtypes = [P, I, I, I, I, I]
         l.spite_attn_prefill_workspace.restype = c_size_t
+        l.spite_delta_chunk_workspace.argtypes = [I, I, I, I]
+        l.spite_delta_chunk_workspace.restype = c_size_t
         l.spite_cu_count.argtypes = []
         l.spite_cu_count.restype = c_int
         _lib = l
@@ -1298,3 +1302,46 @@ def delta_scan(q, k, v, qk_scale, gates, state, out, cu_seqlens, seq_slots, n_se
                                   _ptr(state, "state", f), state.shape[0], _ptr(cu_seqlens, "cu_seqlens", torch.int32),
                                   _ptr(seq_slots, "seq_slots", torch.int32), int(n_seqs), _ptr(out, "out", f), H, G, D, V,
                                   int(bool(single)), _stream()), "delta_scan")
+
+
+DELTA_CHUNK = 32      # tokens a chunk of ``delta_chunk``
+
+
+def delta_chunk_ok(dtype, G, H, D, V) -> bool:
+    """Whether ``delta_chunk`` takes heads of these sizes, q, k and v being column ranges of one row [G*D | G*D | H*V]."""
+    return dtype == torch.bfloat16 and D in (32, 64, 96, 128) and (2 * G * D + H * V) % 8 == 0
+
+
+def delta_chunks(counts, cu_seqlens):
+    """(int32 array, number of chunks): every entry's tokens in runs of ``DELTA_CHUNK`` from its first one: [n + 1] the
+    first chunk of every entry, then the chunks' first tokens, then their lengths."""
+    counts = np.asarray(counts, dtype=np.int64)
+    per = -(-counts // DELTA_CHUNK)
+    first = np.concatenate([[0], np.cumsum(per)])
+    n = int(first[-1])
+    entry = np.repeat(np.arange(len(counts)), per)
+    at = (np.arange(n) - first[entry]) * DELTA_CHUNK
+    return np.concatenate([first, np.asarray(cu_seqlens, dtype=np.int64)[entry] + at,
+                           np.minimum(counts[entry] - at, DELTA_CHUNK)]).astype(np.int32), n
+
+
+def delta_chunk_workspace(n_chunks, G, H, D) -> int:
+    """Bytes of scratch that delta_chunk needs."""
+    if lib().spite_delta_chunk_tokens() != DELTA_CHUNK:
+        raise KernelError("delta_chunk: the library's chunk differs from this module's")
+    return int(lib().spite_delta_chunk_workspace(int(n_chunks), H, G, D))
+
+
+def delta_chunk(q, k, v, qk_scale, gates, state, out, chunks, n_chunks, seq_slots, n_seqs, scratch, G, H, D, V):
+    """``delta_scan`` for bfloat16 rows in chunks of tokens on the matrix units (see delta_rule.hip).  ``chunks`` (int32 on
+    the GPU), ``n_chunks``: what ``delta_chunks`` returns for the step; ``scratch``: a uint8 tensor of
+    ``delta_chunk_workspace`` bytes."""
+    (pq, ldq), (pk, ldk), (pv, ldv) = _delta_checks(q, k, v, qk_scale, gates, state, out, G, H, D, V, "delta_chunk")
+    if q.dtype != torch.bfloat16:
+        raise KernelError(f"delta_chunk: rows of {q.dtype}")
+    if chunks.numel() < n_seqs + 1 + 2 * n_chunks or seq_slots.numel() < n_seqs or scratch.numel() < delta_chunk_workspace(n_chunks, G, H, D):
+        raise KernelError("delta_chunk: metadata or scratch too small")
+    f = torch.float32
+    _check(lib().spite_delta_chunk(pq, pk, pv, ldq, ldk, ldv, _ptr(qk_scale, "qk_scale", f), _ptr(gates, "gates", f), _ptr(state, "state", f),
+                                   state.shape[0], _ptr(chunks, "chunks", torch.int32), int(n_chunks), _ptr(seq_slots, "seq_slots", torch.int32),
+                                   int(n_seqs), _ptr(scratch, "scratch", torch.uint8), _ptr(out, "out", f), H, G, D, V, _stream()), "delta_chunk")

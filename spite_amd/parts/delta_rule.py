@@ -17,13 +17,25 @@ convolution's results take the run's dtype.
 """
 from __future__ import annotations
 
+import numpy as np
 import torch
 
-from .base import Mixer, ParamSpec, CacheNeed, StateNeed, register
+from .base import Mixer, ParamSpec, CacheNeed, StateNeed, register, register_step_array
 from .linear import linear, Weight
 from ..csrc import hipops
 
 UNIT_EPS = 1e-6      # under the root of a unit vector's length
+
+
+def _chunks(host):
+    """The step's tokens in chunks for the matrix-unit kernel; a step of single tokens runs without them."""
+    if int(host.counts.max(initial=1)) <= 1:
+        return np.zeros(0, dtype=np.int32), 0
+    return hipops.delta_chunks(host.counts, host.cu_seqlens)
+
+
+CHUNKS = "delta_rule.chunks"
+register_step_array(CHUNKS, _chunks)
 
 
 @register("mixer", "delta_rule")
@@ -41,6 +53,8 @@ class DeltaRule(Mixer):
         if not 1 <= self.taps <= 32:
             raise ValueError(f"delta_rule: a convolution of {self.taps} taps (1 to 32)")
         self.n_conv = 2 * self.G * self.D + self.H * self.V
+        self.mfma = hipops.delta_chunk_ok(env.dtype, self.G, self.H, self.D, self.V)
+        self.step_arrays = (CHUNKS,) if self.mfma else ()
         self.w_in = self.w_conv = self.a_log = self.dt_bias = self.w_norm = self.wo = None
 
     # ------------------------------------------------------------------ tensors
@@ -73,6 +87,9 @@ class DeltaRule(Mixer):
     def slow_paths(self, page_size):
         notes = []
         if self.env.dtype == torch.bfloat16 and self.w_in is not None:
+            if not self.mfma:
+                notes.append(f"the delta rule runs token by token: {self.D} key channels a head in rows of {self.n_conv} (the matrix-unit kernel "
+                             f"takes 32, 64, 96 or 128 in rows of a multiple of 8)")
             notes += self.w_in.slow_reason("input projection") + self.wo.slow_reason("output projection")
         return notes
 
@@ -98,7 +115,12 @@ class DeltaRule(Mixer):
         hipops.delta_gates(q, k, proj[:, n + HV:n + HV + H], proj[:, n + HV + H:n + HV + 2 * H], self.a_log, self.dt_bias, qk_scale, gates,
                            G, H, D, q_scale=float(D) ** -0.5, eps=UNIT_EPS)
         o = ws.take((T, HV), torch.float32)
-        hipops.delta_scan(q, k, v, qk_scale, gates, state, o, ctx.cu_seqlens, ctx.seq_slots, ctx.n_seqs, G, H, D, V, single=ctx.decode_only)
+        if self.mfma and not ctx.decode_only:
+            chunks, n_chunks = ctx.derived[CHUNKS]
+            scratch = ws.take((hipops.delta_chunk_workspace(n_chunks, G, H, D),), torch.uint8)
+            hipops.delta_chunk(q, k, v, qk_scale, gates, state, o, chunks, n_chunks, ctx.seq_slots, ctx.n_seqs, scratch, G, H, D, V)
+        else:
+            hipops.delta_scan(q, k, v, qk_scale, gates, state, o, ctx.cu_seqlens, ctx.seq_slots, ctx.n_seqs, G, H, D, V, single=ctx.decode_only)
         y = ws.take((T, HV), x.dtype)
         hipops.gated_group_norm(o, self.w_norm, y, V, self.eps, gate=proj[:, n:n + HV], act="silu")
         out = ws.take((T, self.d), torch.float32)
