@@ -172,7 +172,7 @@ class KernelTimes:
              "qkv_prepare", "attn_wide", "attn_finish", "token_shift", "act_rows",
              "linear_attn_scan", "channel_decay", "gated_group_norm", "scale_rows",
              "add_tanh_norm", "hash_rows", "embed_sum", "causal_conv", "shift_mix", "step_decay", "softcap_rows",
-             "axpby_rows", "concat_rows", "bias_rows")
+             "axpby_rows", "concat_rows", "bias_rows", "delta_gates", "delta_scan", "delta_chunk", "gate_rows")
 
     def __init__(self):
         import torch
@@ -245,6 +245,12 @@ class KernelTimes:
 # values), the experts of the size in groups of four of which three are open, the shared expert behind a gate, the third
 # layer dense.  Ravenex at the same width, heads, latent, experts and dense layer, latent attention in every layer, a cache
 # of its own each, no token rows.
+# ``--design porarax``: the Porarax design beside Tebalorn (recurrent states, one norm for both sublayers, attention, several
+# experts a token weighted by the softmax over the taken) and beside Lumevik (latent attention with a query latent, bounded
+# experts), its two closest existing designs.  Porarax: layers in the order delta, latent attention, delta, attention (a state of
+# heads x 128 x 128 numbers, a q/k head for every two value heads, a convolution of four taps; a latent of 512, a query latent of
+# 1,536, a window of 4,096; heads of 128, a kv head for every four, 64 turning elements, a gate on every element), every layer with
+# the experts of the size and no shared expert.
 DESIGN_SIZES = {
     "2k": dict(width=2048, heads=16, experts=16, top=4, expert_ff=1024, shared_ff=2048, dense_ff=8192),
     "5k": dict(width=5120, heads=40, experts=16, top=2, expert_ff=4096, shared_ff=8192, dense_ff=16384),
@@ -331,7 +337,22 @@ def lumevik_configs(sz, layers, window, vocab):
     return {"lumevik": lumevik, "ravenex": ravenex}
 
 
+def porarax_configs(sz, layers, window, vocab):
+    H = sz["heads"]
+    delta = ("delta", {"heads": H, "kv_heads": max(1, H // 2), "dim": 128, "vdim": 128, "conv": 4})
+    latent = ("latent_attention", {"heads": H, "dim": 128, "vdim": 128, "kv_rank": 512, "q_rank": 1536, "scale": 128 ** -0.5, "mask": {"size": window}})
+    attn = ("attention", {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "rot": {"base": 1000000.0, "dims": 64}})
+    mixers = [delta, latent, delta, attn]
+    moe = {"kind": "moe", "router": {"experts": sz["experts"], "top": sz["top"]}, "expert": {"ff": sz["expert_ff"], "limit": 7.0}}
+    porarax = {"architecture": "Porarax", "vocab": vocab, "width": sz["width"], "norm": {"eps": 1e-6}, "torch_dtype": "bfloat16",
+               "layers": [{"type": mixers[i % 4][0], "mixer": mixers[i % 4][1], "mlp": moe} for i in range(layers)]}
+    return {"porarax": porarax, "tebalorn": tebalorn_configs(sz, layers, window, vocab)["tebalorn"],
+            "lumevik": lumevik_configs(sz, layers, window, vocab)["lumevik"]}
+
+
 def design_configs(sz, layers, window, vocab, design="ravenex"):
+    if design == "porarax":
+        return porarax_configs(sz, layers, window, vocab)
     if design == "lumevik":
         return lumevik_configs(sz, layers, window, vocab)
     if design == "nolapel":
@@ -368,7 +389,7 @@ def design_comparison(args):
     page, V, layers, window = 64, 32768, args.layers or 4, 4096
     batch, context, T = args.batch, args.context, args.prefill_tokens
     rng = np.random.RandomState(0)
-    beside = {"nolapel": "Tebalorn", "lumevik": "Ravenex"}.get(args.design, "Llama 4")
+    beside = {"nolapel": "Tebalorn", "lumevik": "Ravenex", "porarax": "Tebalorn and Lumevik"}.get(args.design, "Llama 4")
     out = {"metric": f"prefill and decode tok/s of the {args.design.capitalize()} design beside {beside} at equal sizes (random weights)",
            "value": None, "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "dtype": args.dtype,
            "higher_is_better": True, "data": "synthetic: random weights, uniform-random token ids, context pages filled with random values",
@@ -697,9 +718,10 @@ def main() -> int:
     ap.add_argument("--workload", default="decode", choices=["decode", "longctx", "serve", "designs"],
                     help="designs: another design (--design) beside Llama 4 at equal sizes (see DESIGN_SIZES)")
     ap.add_argument("--design-sizes", default="2k,5k", help="designs: which of DESIGN_SIZES, comma separated")
-    ap.add_argument("--design", default="ravenex", choices=["ravenex", "pefedra", "tebalorn", "nolapel", "lumevik"],
+    ap.add_argument("--design", default="ravenex", choices=["ravenex", "pefedra", "tebalorn", "nolapel", "lumevik", "porarax"],
                     help="designs: which design runs beside Llama 4 (pefedra: against Llama 4 with dense layers only; "
-                         "nolapel: beside Tebalorn, lumevik: beside Ravenex, their closest existing designs)")
+                         "nolapel: beside Tebalorn, lumevik: beside Ravenex, porarax: beside Tebalorn and Lumevik, their closest "
+                         "existing designs)")
     ap.add_argument("--layers", type=int, default=None, help="fewer layers than the model has (memory or time)")
     ap.add_argument("--batch", type=int, default=8)
     ap.add_argument("--context", type=int, default=4096)

@@ -267,7 +267,8 @@ extern "C" int spite_delta_scan(const void* q, const void* k, const void* v, int
 // R_t = beta_t v_t - beta_t exp(G_t) S0^T k_t.  Every exponent is a sum of logarithms of decays, never above 0.
 //
 // The first kernel forms, for every chunk and head at once, what does not depend on the state: (I + A)^-1 (by substitution),
-// the matrix M of the second line and the factors of the rows; and K^T in operand order.  The second walks a head's chunks.
+// the matrix M of the second line and the factors of the rows; and K, Q and K^T in operand order, zeros behind a chunk's
+// last token.  The second walks a head's chunks: it copies what the first has left straight into LDS, a chunk ahead.
 //
 // Nothing is rounded to bfloat16 on the way: K and Q *are* bfloat16 (their factors are applied to the products' rows),
 // and an fp32 operand that meets them (the state, U) is split into three bfloat16 summands, 8 bits each, that add up to
@@ -280,9 +281,10 @@ extern "C" int spite_delta_scan(const void* q, const void* k, const void* v, int
 // supplies as the right operand of the next product: the state never moves between lanes.  The same holds for U (a
 // lane's 4 + 4 tokens): its products take their tokens in the order in which the lanes hold them.
 #define DC_C 32                                      // tokens a chunk
+#define DC_NW 4                                      // waves a workgroup of the walk
 #define DC_TILE 256                                  // floats of a 16 x 16 tile
-#define DC_REC (6 * DC_TILE + 4 * DC_C + 8)          // a chunk's and head's record: inverse and M, three tiles each
-                                                     // (0,0) (1,0) (1,1), the rows' factors, exp(G_C)
+#define DC_REC (7 * DC_TILE)                         // a chunk's and head's record: inverse and M, three tiles each
+                                                     // (0,0) (1,0) (1,1), the rows' factors, exp(G_C); whole kilobytes
 typedef unsigned dc_u4 __attribute__((ext_vector_type(4)));
 
 // element (t, s) of a 16 x 16 tile in the order of the fp32 products' left operand: lane (s/4, t), register s%4
@@ -293,7 +295,7 @@ template <int KD>
 __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(3)))
 void delta_chunk_prepare_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k, int ldq, int ldk, const float* __restrict__ qk_scale,
                                 const float* __restrict__ gates, const int* __restrict__ chunk_t0, const int* __restrict__ chunk_n,
-                                bf16* __restrict__ kt, float* __restrict__ rec, int H, int G) {
+                                bf16* __restrict__ ops, float* __restrict__ rec, int H, int G) {
     constexpr int D = 32 * KD, LK = D + 8;
     __shared__ __attribute__((aligned(16))) bf16 krow[DC_C * LK];
     __shared__ __attribute__((aligned(16))) float at[DC_C][DC_C + 4];       // A transposed: at[s][t]
@@ -400,105 +402,131 @@ void delta_chunk_prepare_kernel(const bf16* __restrict__ q, const bf16* __restri
         for (int r = 0; r < 4; ++r) out[DC_TILE + dc_pos(4 * a + r, row)] = -z[r];
     }
     if (h % (H / G) == 0) {
-        // K^T as the left operand of the state's update: lane (a, row) of tile (j, tt) holds channel 32 j + 8 (row/4) + 4 tt + row%4
-        // of the tokens 4 a .. 4 a + 3 and 16 + 4 a ..
-        bf16* dst = kt + ((size_t)c * G + g) * (2 * KD * 512);
+        // the operands: K and Q as left operands as this wave holds them, then K^T as the left operand of the state's update:
+        // lane (a, row) of tile (j, tt) holds channel 32 j + 8 (row/4) + 4 tt + row%4 of the tokens 4 a .. 4 a + 3 and 16 + 4 a ..
+        bf16x8* dst = (bf16x8*)(ops + ((size_t)c * G + g) * (6 * KD * 512));
+#pragma unroll
+        for (int ti = 0; ti < 2; ++ti)
+#pragma unroll
+            for (int j = 0; j < KD; ++j) {
+                dst[(ti * KD + j) * 64 + lane] = ka[ti][j];
+                dst[(2 * KD + ti * KD + j) * 64 + lane] = qa[ti][j];
+            }
 #pragma unroll
         for (int x = 0; x < 2 * KD; ++x) {
             const int d = 32 * (x >> 1) + 8 * (row >> 2) + 4 * (x & 1) + (row & 3);
             bf16x8 o;
 #pragma unroll
             for (int e = 0; e < 8; ++e) o[e] = krow[((e & 4) * 4 + 4 * a + (e & 3)) * LK + d];
-            *(bf16x8*)(dst + (x * 64 + lane) * 8) = o;
+            dst[(4 * KD + x) * 64 + lane] = o;
         }
     }
 }
 
-// The three bfloat16 summands of eight fp32 numbers.
+// The three bfloat16 summands of eight fp32 numbers: the upper halves of what is left, cut off, 8 bits at a time.
 __device__ __forceinline__ void dc_split(const f32x4& x, const f32x4& y, bf16x8& hi, bf16x8& mid, bf16x8& lo) {
+    dc_u4 h, m, l;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-        const float v = e < 4 ? x[e & 3] : y[e & 3];
-        hi[e] = (bf16)v;
-        const float r = v - (float)hi[e];
-        mid[e] = (bf16)r;
-        lo[e] = (bf16)(r - (float)mid[e]);
+    for (int i = 0; i < 4; ++i) {
+        const float v0 = i < 2 ? x[2 * i & 3] : y[2 * i & 3], v1 = i < 2 ? x[(2 * i + 1) & 3] : y[(2 * i + 1) & 3];
+        const float r0 = v0 - __uint_as_float(__float_as_uint(v0) & 0xffff0000u), r1 = v1 - __uint_as_float(__float_as_uint(v1) & 0xffff0000u);
+        const float s0 = r0 - __uint_as_float(__float_as_uint(r0) & 0xffff0000u), s1 = r1 - __uint_as_float(__float_as_uint(r1) & 0xffff0000u);
+        h[i] = __builtin_amdgcn_perm(__float_as_uint(v1), __float_as_uint(v0), 0x07060302u);     // two upper halves in one register
+        m[i] = __builtin_amdgcn_perm(__float_as_uint(r1), __float_as_uint(r0), 0x07060302u);
+        l[i] = __builtin_amdgcn_perm(__float_as_uint(s1), __float_as_uint(s0), 0x07060302u);
     }
+    hi = __builtin_bit_cast(bf16x8, h);
+    mid = __builtin_bit_cast(bf16x8, m);
+    lo = __builtin_bit_cast(bf16x8, l);
 }
 
-// 256 threads take 64 value columns of one head of one entry, a wave 16 of them, and walk the entry's chunks; the next
-// chunk's operands are on their way in registers while this one is computed from LDS.
+// Four waves take 16 value columns each of one head of one entry and walk the entry's chunks; the next chunk's operands are
+// on their way into the other LDS buffer while this one is computed.
 template <int KD>
-__global__ __launch_bounds__(256)
-void delta_chunk_scan_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k, const bf16* __restrict__ v, int ldq, int ldk, int ldv,
-                             const int* __restrict__ first_chunk, const int* __restrict__ chunk_t0, const int* __restrict__ chunk_n,
-                             const bf16* __restrict__ kt, const float* __restrict__ rec, float* __restrict__ state,
-                             const int* __restrict__ seq_slots, float* __restrict__ out, int H, int G, int V) {
-    constexpr int D = 32 * KD, NO = 128 * KD;             // 16-byte pieces of one operand (K, Q, K^T)
-    constexpr int PIECES = 3 * NO + DC_REC / 4, NP = (PIECES + 255) / 256;
-    static_assert(DC_REC % 4 == 0, "a record is whole pieces");
-    __shared__ __attribute__((aligned(16))) dc_u4 lds[PIECES];
-    const int e = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, a = lane >> 4;
-    const int g = h / (H / G), col = blockIdx.z * 64 + (tid >> 6) * 16 + (lane & 15);
-    const bool cok = col < V;
-    const bool busy = blockIdx.z * 64 + (tid >> 6) * 16 < V;        // the wave has a column at all
+__global__ __launch_bounds__(64 * DC_NW) __attribute__((amdgpu_waves_per_eu(2)))
+void delta_chunk_scan_kernel(const bf16* __restrict__ v, int ldv, const int* __restrict__ first_chunk, const int* __restrict__ chunk_t0,
+                             const int* __restrict__ chunk_n, const bf16* __restrict__ ops, const float* __restrict__ rec,
+                             float* __restrict__ state, const int* __restrict__ seq_slots, float* __restrict__ out, int H, int G, int V) {
+    constexpr int D = 32 * KD, TILES = 6 * KD + 7;         // kilobytes a chunk: K, Q, K^T, the record
+    __shared__ __attribute__((aligned(16))) dc_u4 lds[2][TILES * 64];
+    const int e = blockIdx.x, h = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, a = lane >> 4;
+    const int g = h / (H / G), col0 = (blockIdx.z * DC_NW + wave) * 16 + (lane & 15);
+    const bool cok = col0 < V;
+    const int col = cok ? col0 : V - 1;                    // a lane without a column of its own reads the last one and writes none
     const int c_lo = first_chunk[e], c_hi = first_chunk[e + 1];
     if (c_lo >= c_hi) return;
+    const int t_lo = chunk_t0[c_lo], t_hi = chunk_t0[c_hi - 1] + chunk_n[c_hi - 1];
     float* sbase = state + ((size_t)seq_slots[e] * H + h) * (size_t)D * V + col;
     f32x4 S[2 * KD];
 #pragma unroll
     for (int x = 0; x < 2 * KD; ++x)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[x][r] = cok ? sbase[(size_t)(32 * (x >> 1) + 8 * a + 4 * (x & 1) + r) * V] : 0.f;
-    dc_u4 st[NP];
-    float vn[2][4];
-    // operands of chunk c on their way: K and Q rows in the order of a product's left operand, K^T and the record as they lie
-#define DC_FETCH(c)                                                                                                     \
+        for (int r = 0; r < 4; ++r) S[x][r] = sbase[(size_t)(32 * (x >> 1) + 8 * a + 4 * (x & 1) + r) * V];
+    bf16 vn[2][4];
+    const unsigned v_lane = 4u * a * (unsigned)ldv + col, o_lane = 4u * a * (unsigned)(H * V) + col;    // a lane's tokens 4 a ..
+    // a chunk's operands into an LDS buffer (a wave a kilobyte at a time), its values into registers; tokens behind the last
+    // one read that one's values, which their step size of zero takes out
+#define DC_FETCH(c, buf)                                                                                                \
     {                                                                                                                   \
-        const int t0 = chunk_t0[c], n = chunk_n[c];                                                                     \
+        const dc_u4* so = (const dc_u4*)(ops + ((size_t)(c) * G + g) * (6 * KD * 512)) + lane;                          \
+        const dc_u4* sr = (const dc_u4*)(rec + ((size_t)(c) * H + h) * DC_REC) + lane;                                  \
         _Pragma("unroll")                                                                                               \
-        for (int u = 0; u < NP; ++u) {                                                                                  \
-            const int p = tid + u * 256;                                                                                \
-            if (p < 2 * NO) {                                                                                           \
-                const int o = p % NO, i = 16 * (o / (64 * KD)) + (o & 15), d = 32 * ((o >> 6) % KD) + 8 * ((o >> 4) & 3); \
-                const bool ok = i < n;                                                                                  \
-                const size_t t = t0 + (ok ? i : 0);                                                                     \
-                const dc_u4 got = *(const dc_u4*)((p < NO ? k + t * ldk : q + t * ldq) + (size_t)g * D + d);             \
-                st[u] = ok ? got : dc_u4{0, 0, 0, 0};                                                                   \
-            } else if (p < 3 * NO) {                                                                                    \
-                st[u] = *((const dc_u4*)(kt + ((size_t)(c) * G + g) * (2 * KD * 512)) + (p - 2 * NO));                   \
-            } else if (p < PIECES) {                                                                                    \
-                st[u] = *((const dc_u4*)(rec + ((size_t)(c) * H + h) * DC_REC) + (p - 3 * NO));                          \
+        for (int u = 0; u < (TILES + DC_NW - 1) / DC_NW; ++u) {                                                               \
+            const int x = u * DC_NW + wave;                                                                                \
+            if (x < TILES)                                                                                              \
+                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(x < 6 * KD ? so + x * 64 : sr + (x - 6 * KD) * 64), \
+                                                 (__attribute__((address_space(3))) void*)(lds[buf] + x * 64), 16, 0, 0); \
+        }                                                                                                               \
+        const int t0 = t_lo + ((c) - c_lo) * DC_C;                                                                      \
+        if (t0 + DC_C <= t_hi) {                                                                                        \
+            const bf16* vb = v + (size_t)t0 * ldv + (size_t)h * V;                                                      \
+            _Pragma("unroll")                                                                                           \
+            for (int x = 0; x < 8; ++x) vn[x >> 2][x & 3] = (vb + (size_t)(16 * (x >> 2) + (x & 3)) * ldv)[v_lane];      \
+        } else {                                                                                                        \
+            _Pragma("unroll")                                                                                           \
+            for (int x = 0; x < 8; ++x) {                                                                               \
+                const int t = t0 + 16 * (x >> 2) + 4 * a + (x & 3);                                                     \
+                vn[x >> 2][x & 3] = v[(size_t)(t < t_hi ? t : t_hi - 1) * ldv + (size_t)h * V + col];                   \
             }                                                                                                           \
         }                                                                                                               \
-        _Pragma("unroll")                                                                                               \
-        for (int x = 0; x < 8; ++x) {                                                                                   \
-            const int i = 16 * (x >> 2) + 4 * a + (x & 3);                                                              \
-            const bool ok = i < n && cok;                                                                               \
-            const bf16 got = v[(size_t)(t0 + (ok ? i : 0)) * ldv + (size_t)h * V + (ok ? col : 0)];                     \
-            vn[x >> 2][x & 3] = ok ? (float)got : 0.f;                                                                  \
+    }
+    // a chunk's results leave at the start of the next turn: the wait for a chunk's operands never waits for stores just issued
+    f32x4 O[2];
+#define DC_STORE(c)                                                                                                     \
+    {                                                                                                                   \
+        const int t0 = t_lo + ((c) - c_lo) * DC_C;                                                                      \
+        if (t0 + DC_C <= t_hi) {                                                                                        \
+            float* ob = out + ((size_t)t0 * H + h) * V;                                                                 \
+            if (cok) {                                                                                                  \
+                _Pragma("unroll")                                                                                       \
+                for (int x = 0; x < 8; ++x) (ob + (size_t)(16 * (x >> 2) + (x & 3)) * H * V)[o_lane] = O[x >> 2][x & 3]; \
+            }                                                                                                           \
+        } else {                                                                                                        \
+            _Pragma("unroll")                                                                                           \
+            for (int x = 0; x < 8; ++x) {                                                                               \
+                const int t = t0 + 16 * (x >> 2) + 4 * a + (x & 3);                                                     \
+                if (t < t_hi && cok) out[(size_t)t * H * V + (size_t)h * V + col] = O[x >> 2][x & 3];                   \
+            }                                                                                                           \
         }                                                                                                               \
     }
-    DC_FETCH(c_lo)
-    const bf16x8* kop = (const bf16x8*)lds;
-    const bf16x8* qop = kop + NO;
-    const bf16x8* ktop = qop + NO;
-    const f32x4* inv = (const f32x4*)(lds + 3 * NO);
-    const f32x4* mm = inv + 3 * 64;
-    const f32x4* fr = mm + 3 * 64;                         // the rows' factors, four tokens each
+    DC_FETCH(c_lo, 0)
     for (int c = c_lo; c < c_hi; ++c) {
-        __syncthreads();                                   // the chunk before has been read
-#pragma unroll
-        for (int u = 0; u < NP; ++u) if (tid + u * 256 < PIECES) lds[tid + u * 256] = st[u];
+        const int buf = (c - c_lo) & 1;
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         f32x4 vv[2];
 #pragma unroll
-        for (int x = 0; x < 8; ++x) vv[x >> 2][x & 3] = vn[x >> 2][x & 3];
-        __syncthreads();
-        const int t0 = chunk_t0[c], n = chunk_n[c];
-        if (c + 1 < c_hi) DC_FETCH(c + 1)
-        if (!busy) continue;
+        for (int x = 0; x < 8; ++x) vv[x >> 2][x & 3] = (float)vn[x >> 2][x & 3];
+        __syncthreads();                                   // this chunk has come, the one before has been read
+        if (c > c_lo) DC_STORE(c - 1)
+        if (c + 1 < c_hi) DC_FETCH(c + 1, buf ^ 1)
+        const bf16x8* kop = (const bf16x8*)lds[buf] + lane;
+        const bf16x8* qop = kop + 2 * KD * 64;
+        const bf16x8* ktop = qop + 2 * KD * 64;
+        const f32x4* inv = (const f32x4*)(lds[buf] + 6 * KD * 64);
+        const f32x4* mm = inv + 3 * 64;
+        const f32x4* fr = mm + 3 * 64;                     // the rows' factors, four tokens each
         // S0^T k and S0^T q, the smallest summands first
-        f32x4 R[2], O[2];
+        f32x4 R[2];
 #pragma unroll
         for (int i = 0; i < 2; ++i) { R[i] = f32x4{0.f, 0.f, 0.f, 0.f}; O[i] = R[i]; }
 #pragma unroll
@@ -509,8 +537,8 @@ void delta_chunk_scan_kernel(const bf16* __restrict__ q, const bf16* __restrict_
             for (int y = 0; y < 3; ++y)
 #pragma unroll
                 for (int i = 0; i < 2; ++i) {
-                    R[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kop[(i * KD + j) * 64 + lane], s3[y], R[i], 0, 0, 0);
-                    O[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qop[(i * KD + j) * 64 + lane], s3[y], O[i], 0, 0, 0);
+                    R[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kop[(i * KD + j) * 64], s3[y], R[i], 0, 0, 0);
+                    O[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qop[(i * KD + j) * 64], s3[y], O[i], 0, 0, 0);
                 }
         }
 #pragma unroll
@@ -551,19 +579,16 @@ void delta_chunk_scan_kernel(const bf16* __restrict__ q, const bf16* __restrict_
         dc_split(U[0], U[1], u3[2], u3[1], u3[0]);
         const float whole = fr[32][0];
 #pragma unroll
-        for (int x = 0; x < 2 * KD; ++x) {
-            const bf16x8 w = ktop[x * 64 + lane];
+        for (int x = 0; x < 2 * KD; ++x)
 #pragma unroll
             for (int r = 0; r < 4; ++r) S[x][r] *= whole;
 #pragma unroll
-            for (int y = 0; y < 3; ++y) S[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, u3[y], S[x], 0, 0, 0);
-        }
+        for (int y = 0; y < 3; ++y)
 #pragma unroll
-        for (int x = 0; x < 8; ++x) {
-            const int i = 16 * (x >> 2) + 4 * a + (x & 3);
-            if (i < n && cok) out[(size_t)(t0 + i) * H * V + (size_t)h * V + col] = O[x >> 2][x & 3];
-        }
+            for (int x = 0; x < 2 * KD; ++x) S[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ktop[x * 64], u3[y], S[x], 0, 0, 0);
     }
+    DC_STORE(c_hi - 1)
+#undef DC_STORE
 #undef DC_FETCH
     if (!cok) return;
 #pragma unroll
@@ -572,9 +597,9 @@ void delta_chunk_scan_kernel(const bf16* __restrict__ q, const bf16* __restrict_
         for (int r = 0; r < 4; ++r) sbase[(size_t)(32 * (x >> 1) + 8 * a + 4 * (x & 1) + r) * V] = S[x][r];
 }
 
-// Bytes of scratch for n_chunks chunks: K^T in operand order, then the records.
+// Bytes of scratch for n_chunks chunks: the operands, then the records.
 extern "C" size_t spite_delta_chunk_workspace(int n_chunks, int H, int G, int D) {
-    return (size_t)n_chunks * ((size_t)G * D * DC_C * sizeof(bf16) + (size_t)H * DC_REC * sizeof(float));
+    return (size_t)n_chunks * ((size_t)G * 3 * D * DC_C * sizeof(bf16) + (size_t)H * DC_REC * sizeof(float));
 }
 extern "C" int spite_delta_chunk_tokens() { return DC_C; }
 
@@ -585,18 +610,18 @@ extern "C" int spite_delta_chunk(const void* q, const void* k, const void* v, in
     SP_REQUIRE(n_seqs >= 0 && n_chunks >= 0 && H > 0 && G > 0 && H % G == 0 && V > 0 && n_slots > 0, "delta_chunk: bad sizes H=%d G=%d V=%d", H, G, V);
     SP_REQUIRE(D == 32 || D == 64 || D == 96 || D == 128, "delta_chunk: %d key channels a head (32, 64, 96 or 128)", D);
     SP_REQUIRE(ldq >= G * D && ldk >= G * D && ldv >= H * V, "delta_chunk: rows shorter than the heads");
-    SP_REQUIRE(H <= 65535 && (V + 63) / 64 <= 65535, "delta_chunk: too many heads or value columns");
+    SP_REQUIRE(H <= 65535 && V <= 65535, "delta_chunk: too many heads or value columns");
     auto on16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
     SP_REQUIRE(ldq % 8 == 0 && ldk % 8 == 0 && on16(q) && on16(k) && on16(scratch), "delta_chunk: q and k rows must start on 16 bytes");
     if (n_seqs == 0 || n_chunks == 0) return 0;
-    bf16* kt = (bf16*)scratch;
-    float* rec = (float*)(kt + (size_t)n_chunks * G * D * DC_C);
+    bf16* ops = (bf16*)scratch;
+    float* rec = (float*)(ops + (size_t)n_chunks * G * 3 * D * DC_C);
     const int *first = chunks, *t0 = chunks + n_seqs + 1, *n = t0 + n_chunks;
 #define DC_RUN(KD) do { \
-        delta_chunk_prepare_kernel<KD><<<dim3(n_chunks, H), 64, 0, st>>>((const bf16*)q, (const bf16*)k, ldq, ldk, qk_scale, gates, t0, n, kt, rec, H, G); \
+        delta_chunk_prepare_kernel<KD><<<dim3(n_chunks, H), 64, 0, st>>>((const bf16*)q, (const bf16*)k, ldq, ldk, qk_scale, gates, t0, n, ops, rec, H, G); \
         SP_LAUNCH_CHECK("delta_chunk_prepare"); \
-        delta_chunk_scan_kernel<KD><<<dim3(n_seqs, H, (V + 63) / 64), 256, 0, st>>>((const bf16*)q, (const bf16*)k, (const bf16*)v, ldq, ldk, ldv, \
-            first, t0, n, kt, rec, state, seq_slots, out, H, G, V); } while (0)
+        delta_chunk_scan_kernel<KD><<<dim3(n_seqs, H, (V + 16 * DC_NW - 1) / (16 * DC_NW)), 64 * DC_NW, 0, st>>>( \
+            (const bf16*)v, ldv, first, t0, n, ops, rec, state, seq_slots, out, H, G, V); } while (0)
     if (D == 32) DC_RUN(1); else if (D == 64) DC_RUN(2); else if (D == 96) DC_RUN(3); else DC_RUN(4);
 #undef DC_RUN
     SP_LAUNCH_CHECK("delta_chunk");

@@ -3,7 +3,7 @@
 ``token_table`` (crates/spite-models/src/llama/llama4.rs:118-119): row ``id`` of the table as
 the residual stream's first value, in fp32, times ``scale`` if the architecture has one.
 ``linear_head`` (llama4.rs:277-279): logits = W . (normed last hidden state), W ``[V, d]``;
-tied, it reads the embedding's table; times ``scale`` if the architecture has one; with ``softcap`` c the
+tied, W is the embedding's table; times ``scale`` if the architecture has one; with ``softcap`` c the
 logits become c * tanh(logits / c).  Another architecture's embedding scale, logit cap or
 bias is another kind registered under these categories, not a change to the model class.
 
@@ -87,9 +87,11 @@ class LinearHead(Head):
             self.weight = Weight(tensors["weight"])
 
     def tie(self, embedding):
-        """Tied: the table stays row-major (the embedding reads its rows) and serves as W."""
+        """Tied: W is the embedding's table.  The embedding reads rows, the product reads operand order (its stream of a
+        row-major W takes 1.3 times as long), so where the sizes allow that order the head keeps a copy in it."""
         if self.tied:
-            self.weight = embedding.table
+            w = Weight(embedding.table)
+            self.weight = w if w.tiled else embedding.table
 
     def slow_paths(self, page_size):
         return self.weight.slow_reason("output matrix") if isinstance(self.weight, Weight) else []
