@@ -18,6 +18,15 @@
 #define DR_MAXD 256
 
 // ------------------------------------------------------------------ factors, decays, step sizes
+template <typename T>
+__device__ __forceinline__ void delta_gate(const T* raw_a, int lda, const T* raw_b, int ldb, const float* a_log, const float* dt_bias,
+                                           float* gates, size_t t, int h, int H) {
+    const float z = to_f32<T>(raw_a[t * lda + h]) + dt_bias[h];
+    const float step = z > 20.f ? z + log1pf(expf(-z)) : log1pf(expf(z));           // softplus
+    gates[t * 2 * H + h] = -expf(a_log[h]) * step;
+    gates[t * 2 * H + H + h] = 1.0f / (1.0f + expf(-to_f32<T>(raw_b[t * ldb + h])));
+}
+
 // A wave takes one q/k head of a token (both sums of squares) or, the last item of a token, the heads' decays and
 // step sizes.  qk_scale [T][2][G]: q's factor q_scale / sqrt(sum q^2 + eps), then k's; gates [T][2][H]: log g, then beta.
 template <typename T>
@@ -47,12 +56,40 @@ void delta_gates_kernel(const T* __restrict__ q, const T* __restrict__ k, int ld
         }
         return;
     }
-    for (int h = lane; h < H; h += 64) {
-        const float z = to_f32<T>(raw_a[t * lda + h]) + dt_bias[h];
-        const float step = z > 20.f ? z + log1pf(expf(-z)) : log1pf(expf(z));           // softplus
-        gates[t * 2 * H + h] = -expf(a_log[h]) * step;
-        gates[t * 2 * H + H + h] = 1.0f / (1.0f + expf(-to_f32<T>(raw_b[t * ldb + h])));
+    for (int h = lane; h < H; h += 64) delta_gate(raw_a, lda, raw_b, ldb, a_log, dt_bias, gates, t, h, H);
+}
+
+// The same for bfloat16 rows that a lane reads 16 bytes at a time: 16 lanes a q/k head, four heads a wave (the token's last
+// items are its decays and step sizes).
+__global__ __launch_bounds__(256)
+void delta_gates_vec_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k, int ldq, int ldk, const bf16* __restrict__ raw_a, int lda,
+                            const bf16* __restrict__ raw_b, int ldb, const float* __restrict__ a_log, const float* __restrict__ dt_bias,
+                            float q_scale, float eps, float* __restrict__ qk_scale, float* __restrict__ gates, int Tn, int G, int H, int D) {
+    const int l = threadIdx.x & 15;
+    const int per = G + (H + 15) / 16;                          // items a token: heads, then runs of 16 value heads
+    const size_t item = (size_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+    if (item >= (size_t)Tn * per) return;
+    const size_t t = item / per;
+    const int g = (int)(item - t * per);
+    if (g < G) {
+        const bf16* qr = q + t * ldq + (size_t)g * D;
+        const bf16* kr = k + t * ldk + (size_t)g * D;
+        float sq = 0.f, sk = 0.f;
+        for (int c = l * 8; c < D; c += 128) {
+            const bf16x8 x = *(const bf16x8*)(qr + c), y = *(const bf16x8*)(kr + c);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) { sq = fmaf((float)x[e], (float)x[e], sq); sk = fmaf((float)y[e], (float)y[e], sk); }
+        }
+        sq = row16_sum(sq);
+        sk = row16_sum(sk);
+        if (l == 0) {
+            qk_scale[t * 2 * G + g] = q_scale / sqrtf(sq + eps);
+            qk_scale[t * 2 * G + G + g] = 1.0f / sqrtf(sk + eps);
+        }
+        return;
     }
+    const int h = (g - G) * 16 + l;
+    if (h < H) delta_gate(raw_a, lda, raw_b, ldb, a_log, dt_bias, gates, t, h, H);
 }
 
 extern "C" int spite_delta_gates(const void* q, const void* k, int ldq, int ldk, const void* raw_a, int lda, const void* raw_b, int ldb,
@@ -61,6 +98,15 @@ extern "C" int spite_delta_gates(const void* q, const void* k, int ldq, int ldk,
     SP_REQUIRE(T >= 0 && G > 0 && H > 0 && D > 0 && eps > 0.f, "delta_gates: bad sizes T=%d G=%d H=%d D=%d", T, G, H, D);
     SP_REQUIRE(ldq >= G * D && ldk >= G * D && lda >= H && ldb >= H, "delta_gates: rows shorter than the heads");
     if (T == 0) return 0;
+    auto on16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    if (dtype == SP_BF16 && D % 8 == 0 && ldq % 8 == 0 && ldk % 8 == 0 && on16(q) && on16(k)) {
+        const size_t n = (size_t)T * (G + (H + 15) / 16);
+        SP_REQUIRE((n + 15) / 16 < (1u << 31), "delta_gates: too many heads");
+        delta_gates_vec_kernel<<<(unsigned)((n + 15) / 16), 256, 0, st>>>((const bf16*)q, (const bf16*)k, ldq, ldk, (const bf16*)raw_a, lda,
+            (const bf16*)raw_b, ldb, a_log, dt_bias, q_scale, eps, qk_scale, gates, T, G, H, D);
+        SP_LAUNCH_CHECK("delta_gates");
+        return 0;
+    }
     const size_t items = (size_t)T * (G + 1);
     SP_REQUIRE((items + 3) / 4 < (1u << 31), "delta_gates: too many heads");
     const unsigned grid = (unsigned)((items + 3) / 4);

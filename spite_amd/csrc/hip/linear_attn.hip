@@ -382,6 +382,49 @@ void gated_group_norm_kernel(const float* __restrict__ o, const TO* __restrict__
     }
 }
 
+// The same for bfloat16 rows in groups of up to 256 that a lane moves eight elements at a time: 16 lanes a group.
+__global__ __launch_bounds__(256)
+void gated_group_norm_vec_kernel(const float* __restrict__ o, const bf16* __restrict__ gate, int ldg, const float* __restrict__ w, int n_w,
+                                 bf16* __restrict__ y, int T, int n, int group, float eps, int act) {
+    const int l = threadIdx.x & 15, groups = n / group;
+    const size_t item = (size_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+    if (item >= (size_t)T * groups) return;
+    const size_t t = item / groups;
+    const int c0 = (int)(item - t * groups) * group;
+    const float* orow = o + t * n + c0;
+    f32x4 x[2][2];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int c = l * 8 + i * 128;
+#pragma unroll
+        for (int p = 0; p < 2; ++p) {
+            x[i][p] = c < group ? *(const f32x4*)(orow + c + 4 * p) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ss = fmaf(x[i][p][e], x[i][p][e], ss);
+        }
+    }
+    const float sc = 1.0f / sqrtf(row16_sum(ss) / (float)group + eps);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int c = l * 8 + i * 128;
+        if (c >= group) continue;
+        const float* wr = w + (c0 + c) % n_w;                  // (a multiple of eight: n_w is one, or a group's multiple)
+        bf16x8 g, out;
+        if (act) g = *(const bf16x8*)(gate + t * ldg + c0 + c);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            float v = x[i][e >> 2][e & 3] * sc * wr[e];
+            if (act) {
+                const float z = (float)g[e], sg = 1.0f / (1.0f + expf(-z));
+                v *= act == 1 ? z * sg : sg;
+            }
+            out[e] = (bf16)v;
+        }
+        *(bf16x8*)(y + t * n + c0 + c) = out;
+    }
+}
+
 // The same for wide groups (the heads normed together): a workgroup a (token, group), the sum of squares across
 // its four waves through LDS.
 template <typename TO>
@@ -431,6 +474,13 @@ extern "C" int spite_gated_group_norm(const float* o, const void* gate, int ldg,
         else if (y_dtype == SP_BF16)
             gated_group_norm_wide_kernel<bf16><<<(unsigned)items, 256, 0, st>>>(o, (const bf16*)gate, ldg, w, n_w, (bf16*)y, n, group, eps, act, ex);
         else return sp_fail("gated_group_norm: unknown dtype %d", y_dtype);
+        SP_LAUNCH_CHECK("gated_group_norm");
+        return 0;
+    }
+    auto on16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    if (y_dtype == SP_BF16 && !skip && !pre_gate && group % 8 == 0 && group <= 256 && n_w % 8 == 0 && on16(o) && on16(y)
+        && (act == 0 || (ldg % 8 == 0 && on16(gate)))) {
+        gated_group_norm_vec_kernel<<<(unsigned)((items + 15) / 16), 256, 0, st>>>(o, (const bf16*)gate, ldg, w, n_w, (bf16*)y, T, n, group, eps, act);
         SP_LAUNCH_CHECK("gated_group_norm");
         return 0;
     }

@@ -471,6 +471,21 @@ def test_gate_kernel(dtype, n, spare):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("dtype,heads,V", [("bfloat16", 5, 48), ("bfloat16", 3, 128), ("bfloat16", 2, 256), ("bfloat16", 2, 264), ("bfloat16", 3, 20), ("float32", 3, 48)])
+def test_head_norm_and_gate_kernel(dtype, heads, V):
+    """Every head on its own, one weight for all, silu of a column range: rows that a lane moves 16 bytes at a time and others."""
+    from spite_amd.csrc import hipops
+    g = torch.Generator().manual_seed(V)
+    dt = getattr(torch, dtype)
+    T, n = 7, heads * V
+    o, w, z = torch.randn(T, n, generator=g), torch.rand(V, generator=g) + 0.5, (torch.randn(T, n + 16, generator=g) * 2).to(dt)
+    y = torch.empty(T, n, dtype=dt, device="cuda:0")
+    hipops.gated_group_norm(o.cuda(), w.cuda(), y, V, 1e-3, gate=z.cuda()[:, 16:], act="silu")
+    want = plain.norm(o.double().view(T, heads, V), w.double(), 1e-3).view(T, n) * plain.silu(z.double()[:, 16:])
+    assert float((y.cpu().double() - want).abs().max()) < (1e-5 if dtype == "float32" else 1e-2) * float(want.abs().max())
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("E,top", [(6, 2), (1, 1), (70, 5), (300, 66), (8, 8)])
 def test_router_kernel(E, top):
     """The bias is part of the logits: in the choice and in the softmax over the taken."""
