@@ -517,8 +517,8 @@ void delta_chunk_scan_kernel(const bf16* __restrict__ v, int ldv, const int* __r
         const dc_u4* so = (const dc_u4*)(ops + ((size_t)(c) * G + g) * (6 * KD * 512)) + lane;                          \
         const dc_u4* sr = (const dc_u4*)(rec + ((size_t)(c) * H + h) * DC_REC) + lane;                                  \
         _Pragma("unroll")                                                                                               \
-        for (int u = 0; u < (TILES + DC_NW - 1) / DC_NW; ++u) {                                                               \
-            const int x = u * DC_NW + wave;                                                                                \
+        for (int u = 0; u < (TILES + DC_NW - 1) / DC_NW; ++u) {                                                         \
+            const int x = u * DC_NW + wave;                                                                             \
             if (x < TILES)                                                                                              \
                 __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(x < 6 * KD ? so + x * 64 : sr + (x - 6 * KD) * 64), \
                                                  (__attribute__((address_space(3))) void*)(lds[buf] + x * 64), 16, 0, 0); \
